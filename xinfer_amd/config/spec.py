@@ -61,11 +61,13 @@ class ScheduleEntry:
     layer that is run again with the same tensors, as a layer of its own: ids and the indices
     of layers that own a cache share one numbering, so an id is no such layer's index).  `before`: a stream op
     (a `PartSpec` of that registry) that runs on the residual stream right before this run, e.g. what a pass over a
-    span of layers adds to the stream when it starts."""
+    span of layers adds to the stream when it starts; `after`: stream ops that run right after it, in order (what a
+    layer gets besides its branches, an average over the layers so far)."""
     layer: int
     cache_of: Optional[int] = None
     cache_id: Optional[int] = None
     before: Optional[PartSpec] = None
+    after: Tuple[PartSpec, ...] = ()
 
 
 @dataclass(frozen=True)

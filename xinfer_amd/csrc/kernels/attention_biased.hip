@@ -9,6 +9,7 @@
 //     and key position j; then the mask (causal, window).  tanh(x) = 1 - 2 / (2^(2 x log2 e) + 1):
 //     one exponential and one reciprocal a score beside the softmax's own exponential, which is
 //     why this kernel spends more of its time outside the matrix cores than the plain one.
+//   - chunks: a query sees no key from before its chunk's first position (chunks counted from position 0);
 //   - a K pool of fewer heads than the V pool (`nkk`, a divisor of nkv: kv head c reads key head c / (nkv / nkk));
 //     one key head of all kv heads' dims side by side serves heads whose scores are mixed.
 // It serves every mix of prompt portions and single tokens (a single token is a block of one
@@ -24,6 +25,13 @@ constexpr float kLog2eB = 1.4426950408889634f;
 constexpr int kKeysB = 64;    // keys per tile (two steps of 32)
 constexpr int kVPadB = 8;     // bf16 elements of padding per LDS row
 constexpr float kSlackB = 8.f;  // how far (log2) a score may exceed the softmax reference point
+
+// the first key a query at `pos` sees (a window of 0, chunks of 0: none)
+static __device__ __forceinline__ int first_key(int pos, int window, int chunk) {
+  int lo = (window > 0 && pos - window + 1 > 0) ? pos - window + 1 : 0;
+  if (chunk > 0) lo = max(lo, pos - pos % chunk);
+  return lo;
+}
 
 static __device__ __forceinline__ bf16x8 ld8(const bf16* p) { return *reinterpret_cast<const bf16x8*>(p); }
 static __device__ __forceinline__ void st8(bf16* p, bf16x8 v) { *reinterpret_cast<bf16x8*>(p) = v; }
@@ -47,7 +55,7 @@ __global__ __launch_bounds__(64 * NWV, 2) void attn_biased_lds_kernel(
     const int* __restrict__ cu_q, const int* __restrict__ ctx_lens, bf16* __restrict__ out, float scale,
     float softcap, const float* __restrict__ slopes, const float* __restrict__ sinks, int window, int page_shift, int nq,
     int nkv, int d, int dv, float* __restrict__ part_o, float* __restrict__ part_ml, int split_keys, int max_splits,
-    int rows_heads, int nkk, int rows_kv) {
+    int rows_heads, int nkk, int rows_kv, int chunk) {
   const int page = 1 << page_shift;
   constexpr int NT = 64 * NWV;                    // threads
   constexpr int QB = 16 * (NWV * NQT / GH);       // query positions per workgroup
@@ -94,7 +102,7 @@ __global__ __launch_bounds__(64 * NWV, 2) void attn_biased_lds_kernel(
   // keys the workgroup walks
   const int wg_nq = min(QB, q_len - q0_blk);
   const int wg_first = pos0 + step * q0_blk, wg_last = wg_first + step * (wg_nq - 1);
-  const int wg_lo = (window > 0 && wg_first - window + 1 > 0) ? wg_first - window + 1 : 0;
+  const int wg_lo = first_key(wg_first, window, chunk);
   const int k_begin = wg_lo & ~(kKeysB - 1);
   // split_keys > 0 (steps of single tokens): this workgroup walks one slice of the keys, slice
   // blockIdx.z of `split_keys` keys, and leaves its sums unnormalized for the combine kernel
@@ -126,8 +134,8 @@ __global__ __launch_bounds__(64 * NWV, 2) void attn_biased_lds_kernel(
   const bool active = q0 < q_len;
   const int n_q = active ? min(16 * (pb_hi - pb_lo + 1), q_len - q0) : 0;
   const int first_pos = pos0 + step * q0, last_pos = first_pos + step * (n_q - 1);
-  const int lo_first = (window > 0 && first_pos - window + 1 > 0) ? first_pos - window + 1 : 0;
-  const int lo_last = (window > 0 && last_pos - window + 1 > 0) ? last_pos - window + 1 : 0;
+  const int lo_first = active ? first_key(first_pos, window, chunk) : 0;
+  const int lo_last = active ? first_key(last_pos, window, chunk) : 0;
   const int wave_k_begin = lo_first & ~31;
 
   bf16x8 qb[NQT][KC];
@@ -143,7 +151,7 @@ __global__ __launch_bounds__(64 * NWV, 2) void attn_biased_lds_kernel(
     const int qi = q0_blk + 16 * pb + r;
     const bool ok = active && qi < q_len;
     qpos[ct] = ok ? pos0 + step * qi : -1;
-    qlo[ct] = (ok && window > 0 && qpos[ct] - window + 1 > 0) ? qpos[ct] - window + 1 : 0;
+    qlo[ct] = ok ? first_key(qpos[ct], window, chunk) : 0;
     const bf16* qrow = q + ((size_t)(q_begin + (ok ? qi : 0)) * nq + h0 + hh) * d;
 #pragma unroll
     for (int c = 0; c < KC; ++c) {
@@ -479,7 +487,8 @@ int xi_attention_biased_bf16(const void* q, const void* k_cache, const void* vt_
                              int max_pages, const int* tiles, int n_tiles, const int* cu_q, const int* ctx_lens,
                              void* out, float scale, float softcap, const float* slopes, const float* sinks, int window,
                              int page, int nq, int nkv, int d, int dv, int small, float* part_o, float* part_ml, int split_keys,
-                             int max_splits, int n_tok, int rows_heads, int nkk, int rows_kv, hipStream_t stream) {
+                             int max_splits, int n_tok, int rows_heads, int nkk, int rows_kv, int chunk, hipStream_t stream) {
+  XI_CHECK(window >= 0 && chunk >= 0, "attention_biased: a window of %d and chunks of %d", window, chunk);
   XI_CHECK(rows_kv >= 1 && (rows_kv == 1 || (rows_heads > 0 && rows_heads % rows_kv == 0)),
            "attention_biased: %d value heads for rows that are %d heads", rows_kv, rows_heads);
   XI_CHECK(nkk > 0 && nkv % nkk == 0, "attention_biased: %d kv heads on %d key heads", nkv, nkk);
@@ -518,7 +527,7 @@ int xi_attention_biased_bf16(const void* q, const void* k_cache, const void* vt_
     kern<<<grid, 64 * NWV, lds, stream>>>((const bf16*)q, (const bf16*)k_cache, (const bf16*)vt_cache,  \
                                           block_tables, max_pages, tiles, cu_q, ctx_lens, (bf16*)out,   \
                                           scale, softcap, slopes, sinks, window, page_shift, nq, nkv, d,\
-                                          dv, part_o, part_ml, split_keys, max_splits, rows_heads, nkk, rows_kv);\
+                                          dv, part_o, part_ml, split_keys, max_splits, rows_heads, nkk, rows_kv, chunk);\
   } while (0)
 #define XI_PB_GH(KC, DT, NQT, NWV)             \
   do {                                         \

@@ -2,7 +2,7 @@
 // It serves every case (prompt portions, decode tokens, windows, any head size) and is
 // the attention of the 32-bit path; the bfloat16 path uses it where no faster kernel
 // applies.  Keys of a token at position p are the cached positions lo..p of its own
-// request, lo = max(0, p - window + 1), read through the request's block table.  K is
+// request, lo = max(0, p - window + 1) (with chunks of size c also not before the chunk's first position, p - p mod c), read through the request's block table.  K is
 // [page, kv_head, offset, d]; V is [page, kv_head, offset, dv] or, with v_grouped,
 // [page, kv_head, offset / 8, dv, 8]; the value head size dv may differ from d.
 //
@@ -37,7 +37,7 @@ __global__ __launch_bounds__(kAttnWaves* kWave) void attention_generic_kernel(
     const int* __restrict__ block_tables, int max_pages, const int* __restrict__ tok_seq,
     const int* __restrict__ positions, T* __restrict__ out, float scale, int window, int page_size,
     int nq, int nkv, int d, int dv, int v_grouped, float softcap, const float* __restrict__ slopes,
-    const float* __restrict__ sinks, int values_in_keys, int nkk) {
+    const float* __restrict__ sinks, int values_in_keys, int nkk, int chunk) {
   extern __shared__ float q_s[];       // [d]
   __shared__ float acc_s[kAttnWaves][MAXD];
   __shared__ float m_s[kAttnWaves], l_s[kAttnWaves];
@@ -50,7 +50,8 @@ __global__ __launch_bounds__(kAttnWaves* kWave) void attention_generic_kernel(
   const int wave = threadIdx.x / kWave;
   const int seq = tok_seq[t];
   const int pos = positions[t];
-  const int lo = (window > 0 && pos - window + 1 > 0) ? pos - window + 1 : 0;
+  int lo = (window > 0 && pos - window + 1 > 0) ? pos - window + 1 : 0;
+  if (chunk > 0) lo = max(lo, pos - pos % chunk);
   const int* bt = block_tables + (size_t)seq * max_pages;
 
   const T* qp = q + ((size_t)t * nq + h) * d;
@@ -153,7 +154,7 @@ extern "C" int xi_attention_generic(const void* q, const void* k_cache, const vo
                                     const int* tok_seq, const int* positions, void* out,
                                     float scale, int window, int page_size, int n_tok, int nq,
                                     int nkv, int d, int dv, int v_grouped, float softcap, const float* slopes,
-                                    const float* sinks, int values_in_keys, int nkk, hipStream_t stream) {
+                                    const float* sinks, int values_in_keys, int nkk, int chunk, hipStream_t stream) {
   XI_CHECK(n_tok >= 0 && nq > 0 && nkv > 0 && page_size > 0 && max_pages > 0,
            "attention: bad sizes T=%d nq=%d nkv=%d page=%d max_pages=%d", n_tok, nq, nkv, page_size, max_pages);
   XI_CHECK(nq % nkv == 0, "attention: %d query heads are not a multiple of %d kv heads", nq, nkv);
@@ -161,6 +162,7 @@ extern "C" int xi_attention_generic(const void* q, const void* k_cache, const vo
   XI_CHECK(d > 0 && d <= kMaxKeyDim, "attention: head_dim %d is outside 1..%d", d, kMaxKeyDim);
   XI_CHECK(dv > 0 && dv <= kMaxHeadDimWide, "attention: value head size %d is outside 1..%d", dv, kMaxHeadDimWide);
   XI_CHECK(!values_in_keys || (dv <= d && !v_grouped), "attention: values that are the keys' first dims need dv <= d");
+  XI_CHECK(window >= 0 && chunk >= 0, "attention: a window of %d and chunks of %d", window, chunk);
   XI_CHECK(softcap >= 0.f, "attention: the soft cap must be positive (0: none), got %g", (double)softcap);
   XI_CHECK(nq <= 65535, "attention: too many heads (%d)", nq);
   XI_CHECK(!v_grouped || page_size % 8 == 0, "attention: V in groups of eight keys needs pages of a multiple of 8 tokens, not %d", page_size);
@@ -171,7 +173,7 @@ extern "C" int xi_attention_generic(const void* q, const void* k_cache, const vo
 #define XI_AG(TT, MAXD)                                                                                                 \
   attention_generic_kernel<TT, MAXD><<<grid, kAttnWaves * kWave, q_bytes, stream>>>(                                          \
       (const TT*)q, (const TT*)k_cache, (const TT*)v_cache, block_tables, max_pages, tok_seq, positions, (TT*)out, scale, \
-      window, page_size, nq, nkv, d, dv, v_grouped, softcap, slopes, sinks, values_in_keys, nkk)
+      window, page_size, nq, nkv, d, dv, v_grouped, softcap, slopes, sinks, values_in_keys, nkk, chunk)
   if (dtype == kF32 && !wide) XI_AG(float, kMaxHeadDim);
   else if (dtype == kF32) XI_AG(float, kMaxHeadDimWide);
   else if (dtype == kBF16 && !wide) XI_AG(bf16, kMaxHeadDim);

@@ -78,10 +78,10 @@ __global__ __launch_bounds__(256) void latent_rows_kernel(const T* __restrict__ 
 constexpr int kHlRows = 32, kHlCols = 64, kHlK = 32;
 
 // a workgroup of 256 threads: 32 tokens by 64 outputs of one head; a thread 2 tokens by 4 outputs
-template <typename T>
+template <typename T, typename TO>
 __global__ __launch_bounds__(256) void head_linear_kernel(const T* __restrict__ x, long long x_row, long long x_head,
                                                           const T* __restrict__ w, long long w_head, long long w_n,
-                                                          long long w_k, T* __restrict__ out, long long o_row,
+                                                          long long w_k, TO* __restrict__ out, long long o_row,
                                                           long long o_head, const T* __restrict__ gate, long long g_row,
                                                           long long g_head, int g_each, int n_tok, int N, int K) {
   __shared__ float xs[kHlK][kHlRows + 1];
@@ -136,7 +136,7 @@ __global__ __launch_bounds__(256) void head_linear_kernel(const T* __restrict__ 
         const float g = to_float(gate[(size_t)t * g_row + (size_t)h * g_head + (g_each ? n : 0)]);
         v *= 1.f / (1.f + expf(-g));
       }
-      out[(size_t)t * o_row + (size_t)h * o_head + n] = from_float<T>(v);
+      out[(size_t)t * o_row + (size_t)h * o_head + n] = from_float<TO>(v);
     }
   }
 }
@@ -295,7 +295,7 @@ int xi_latent_rows(const void* proj, long long proj_stride, int q_off, int down_
 // or (g_each 0) one number a head at gate + t g_row + h g_head.
 int xi_head_linear(const void* x, long long x_row, long long x_head, const void* w, long long w_head, long long w_n,
                    long long w_k, void* out, long long o_row, long long o_head, const void* gate, long long g_row,
-                   long long g_head, int g_each, int dtype, int n_tok, int H, int N, int K, hipStream_t stream) {
+                   long long g_head, int g_each, int dtype, int out_dtype, int n_tok, int H, int N, int K, hipStream_t stream) {
   XI_CHECK(n_tok >= 0 && H > 0 && N > 0 && K > 0, "head_linear: bad sizes T=%d H=%d N=%d K=%d", n_tok, H, N, K);
   XI_CHECK(w_n == 1 || w_k == 1, "head_linear: the weight's outputs or its inputs must lie side by side");
   XI_CHECK(H <= 65535, "head_linear: too many heads");
@@ -305,7 +305,8 @@ int xi_head_linear(const void* x, long long x_row, long long x_head, const void*
   // bfloat16 with every operand's inputs side by side in whole 16-byte chunks: the matrix cores
   const bool chunks = K % 8 == 0 && w_k == 1 && x_row % 8 == 0 && x_head % 8 == 0 && w_head % 8 == 0 && w_n % 8 == 0 &&
                       (reinterpret_cast<uintptr_t>(x) & 15) == 0 && (reinterpret_cast<uintptr_t>(w) & 15) == 0;
-  if (dtype == kBF16 && chunks) {
+  XI_CHECK(out_dtype == dtype || out_dtype == kF32, "head_linear: results in the operands' type or float32");
+  if (dtype == kBF16 && out_dtype == kBF16 && chunks) {
     dim3 mgrid((unsigned)((n_tok + kHmRows - 1) / kHmRows), (unsigned)((N + kHmCols - 1) / kHmCols), (unsigned)H);
     // outputs (and the gate) in 8-byte pieces where every lane's 4 outputs start at one
     const int wide = o_row % 4 == 0 && o_head % 4 == 0 && (reinterpret_cast<uintptr_t>(out) & 7) == 0 &&
@@ -317,11 +318,15 @@ int xi_head_linear(const void* x, long long x_row, long long x_head, const void*
     return 0;
   }
   if (dtype == kF32)
-    head_linear_kernel<float><<<grid, 256, 0, stream>>>((const float*)x, x_row, x_head, (const float*)w, w_head, w_n, w_k,
+    head_linear_kernel<float, float><<<grid, 256, 0, stream>>>((const float*)x, x_row, x_head, (const float*)w, w_head, w_n, w_k,
                                                         (float*)out, o_row, o_head, (const float*)gate, g_row, g_head, g_each,
                                                         n_tok, N, K);
+  else if (dtype == kBF16 && out_dtype == kF32)
+    head_linear_kernel<bf16, float><<<grid, 256, 0, stream>>>((const bf16*)x, x_row, x_head, (const bf16*)w, w_head, w_n, w_k,
+                                                              (float*)out, o_row, o_head, (const bf16*)gate, g_row, g_head, g_each,
+                                                              n_tok, N, K);
   else if (dtype == kBF16)
-    head_linear_kernel<bf16><<<grid, 256, 0, stream>>>((const bf16*)x, x_row, x_head, (const bf16*)w, w_head, w_n, w_k,
+    head_linear_kernel<bf16, bf16><<<grid, 256, 0, stream>>>((const bf16*)x, x_row, x_head, (const bf16*)w, w_head, w_n, w_k,
                                                        (bf16*)out, o_row, o_head, (const bf16*)gate, g_row, g_head, g_each, n_tok,
                                                        N, K);
   else

@@ -20,7 +20,7 @@
 // n[c] q[c] once a token (the grid covers the v_cols columns; the first tile's workgroup writes the column).
 // With `group_heads` g > 1, q and k have one set of dk columns for every g heads (head h reads set h / g).
 // q, k and v are columns of a packed projection (a row stride and a column offset each); q and k are
-// multiplied by `q_scale` / `k_scale` in float32 as they are read.
+// multiplied by `q_scale` / `k_scale` in float32 as they are read; with `act`, q, k and v pass silu first (float32).
 //
 // `linear_scan_kernel`: one workgroup per (item, head, 64 value columns) walks the item's tokens in order,
 // from a state it is told to start from, and may leave the new state somewhere.  Lane l owns value column l
@@ -66,7 +66,7 @@ __global__ __launch_bounds__(kScanWaves* kWave) void linear_scan_kernel(
     int group_heads, const float* __restrict__ state_in, long long in_stride, const long long* __restrict__ in_idx,
     float* __restrict__ state_out, long long out_stride, const long long* __restrict__ out_idx,
     const int* __restrict__ first, const int* __restrict__ last, float* __restrict__ out, float* __restrict__ decay_out,
-    int H, int dk, int dv, float q_scale, float k_scale) {
+    int H, int dk, int dv, float q_scale, float k_scale, int act) {
   __shared__ __attribute__((aligned(16))) float qs[2][kScanWaves * 64], ks[2][kScanWaves * 64], as[2][kScanWaves * 64];
   __shared__ float part[2][kScanWaves][kScanCols];
   __shared__ float npart[2][kScanWaves];
@@ -98,10 +98,14 @@ __global__ __launch_bounds__(kScanWaves* kWave) void linear_scan_kernel(
     const float x = to_float(step[(size_t)t * step_stride + h]) + sb;
     return fmaxf(x, 0.f) + log1pf(expf(-fabsf(x)));
   };
+  auto read = [&](T x) {
+    const float f = to_float(x);
+    return act ? f / (1.f + expf(-f)) : f;
+  };
   auto fetch = [&](int t, float dt, float& fq, float& fk, float& fa) {      // (channels past the head's stay zero)
     if (c < dk) {
-      fq = to_float(q[(size_t)t * q_stride + qk0 + c]) * q_scale;
-      fk = to_float(k[(size_t)t * k_stride + qk0 + c]) * k_scale;
+      fq = read(q[(size_t)t * q_stride + qk0 + c]) * q_scale;
+      fk = read(k[(size_t)t * k_stride + qk0 + c]) * k_scale;
       if (!ONE) fa = decay_of(z[((size_t)t * H + h) * dk + c] + zb, inv_tau);
     }
     if (ONE) fa = gates ? gates[((size_t)t * H + h) * 2] : step ? expf(rate * dt) : hd;
@@ -111,7 +115,7 @@ __global__ __launch_bounds__(kScanWaves* kWave) void linear_scan_kernel(
   fetch(t0, dt, fq, fk, fa);
   // the token's value is asked for a token ahead as well: no step of the walk waits for memory
   // (a column past the value rows' own reads 1)
-  auto value_of = [&](int t) { return j < v_cols ? to_float(v[(size_t)t * v_stride + h * v_cols + j]) : 1.f; };
+  auto value_of = [&](int t) { return j < v_cols ? read(v[(size_t)t * v_stride + h * v_cols + j]) : 1.f; };
   float v_next = col ? value_of(t0) * dt : 0.f;
   qs[0][c] = fq;
   ks[0][c] = fk;
@@ -218,6 +222,71 @@ __global__ __launch_bounds__(256) void head_norm_gate_kernel(const float* __rest
   }
 }
 
+// What follows the state where the heads are normed together: a row of o divided by its root mean square over all W
+// columns (eps inside the root), times a weight [W], times act(g) (1: sigmoid, 0: silu).  A workgroup a row; VEC: rows in
+// whole pieces of 4, of which a thread keeps its first kRowKeep in registers.
+constexpr int kRowKeep = 4;
+static __device__ __forceinline__ float row_gate(float g, int act) {
+  const float sg = 1.f / (1.f + expf(-g));
+  return act ? sg : g * sg;
+}
+struct alignas(8) rec_bf16x4 { bf16 v[4]; };
+static __device__ __forceinline__ float4 rec_load4(const float* p) { return *reinterpret_cast<const float4*>(p); }
+static __device__ __forceinline__ float4 rec_load4(const bf16* p) {
+  const rec_bf16x4 t = *reinterpret_cast<const rec_bf16x4*>(p);
+  return float4{to_float(t.v[0]), to_float(t.v[1]), to_float(t.v[2]), to_float(t.v[3])};
+}
+static __device__ __forceinline__ void rec_store4(float* p, float4 v) { *reinterpret_cast<float4*>(p) = v; }
+static __device__ __forceinline__ void rec_store4(bf16* p, float4 v) {
+  rec_bf16x4 t;
+  t.v[0] = from_float<bf16>(v.x);
+  t.v[1] = from_float<bf16>(v.y);
+  t.v[2] = from_float<bf16>(v.z);
+  t.v[3] = from_float<bf16>(v.w);
+  *reinterpret_cast<rec_bf16x4*>(p) = t;
+}
+
+template <typename T, int NT, bool VEC>
+__global__ __launch_bounds__(NT) void row_norm_gate_kernel(const float* __restrict__ o, const float* __restrict__ w, float eps,
+                                                           const T* __restrict__ g, long long g_stride, int act,
+                                                           T* __restrict__ out, int W) {
+  __shared__ float scratch[NT / kWave];
+  const size_t t = blockIdx.x;
+  const float* x = o + t * W;
+  const T* gr = g + t * g_stride;
+  T* orow = out + t * W;
+  float ss = 0.f;
+  if constexpr (VEC) {
+    float4 kept[kRowKeep];
+#pragma unroll
+    for (int n = 0; n < kRowKeep; ++n) {
+      const int i = 4 * (n * NT + threadIdx.x);
+      kept[n] = i < W ? rec_load4(x + i) : float4{0.f, 0.f, 0.f, 0.f};
+      ss += (kept[n].x * kept[n].x + kept[n].y * kept[n].y) + (kept[n].z * kept[n].z + kept[n].w * kept[n].w);
+    }
+    for (int i = 4 * (kRowKeep * NT + threadIdx.x); i < W; i += 4 * NT) {
+      const float4 v = rec_load4(x + i);
+      ss += (v.x * v.x + v.y * v.y) + (v.z * v.z + v.w * v.w);
+    }
+    const float inv = rsqrtf(block_sum<NT / kWave>(ss, scratch) / (float)W + eps);
+    auto put = [&](int i, const float4& v) {
+      const float4 wv = rec_load4(w + i), gv = rec_load4(gr + i);
+      rec_store4(orow + i, float4{v.x * inv * wv.x * row_gate(gv.x, act), v.y * inv * wv.y * row_gate(gv.y, act),
+                                  v.z * inv * wv.z * row_gate(gv.z, act), v.w * inv * wv.w * row_gate(gv.w, act)});
+    };
+#pragma unroll
+    for (int n = 0; n < kRowKeep; ++n) {
+      const int i = 4 * (n * NT + threadIdx.x);
+      if (i < W) put(i, kept[n]);
+    }
+    for (int i = 4 * (kRowKeep * NT + threadIdx.x); i < W; i += 4 * NT) put(i, rec_load4(x + i));
+  } else {
+    for (int i = threadIdx.x; i < W; i += NT) ss = fmaf(x[i], x[i], ss);
+    const float inv = rsqrtf(block_sum<NT / kWave>(ss, scratch) / (float)W + eps);
+    for (int i = threadIdx.x; i < W; i += NT) orow[i] = from_float<T>(x[i] * inv * w[i] * row_gate(to_float(gr[i]), act));
+  }
+}
+
 }  // namespace xi
 
 using namespace xi;
@@ -239,7 +308,7 @@ int xi_linear_scan(const void* q, long long q_stride, const void* k, long long k
                    int group_heads, const float* state_in,
                    long long in_stride, const long long* in_idx, float* state_out, long long out_stride,
                    const long long* out_idx, const int* first, const int* last, float* out, float* decay_out, int n_items, int H,
-                   int dk, int dv, float q_scale, float k_scale, hipStream_t stream) {
+                   int dk, int dv, float q_scale, float k_scale, int act, hipStream_t stream) {
   XI_CHECK(n_items >= 0 && H > 0 && dk > 0 && dv > 0, "linear_scan: bad sizes items=%d H=%d dk=%d dv=%d", n_items, H, dk, dv);
   XI_CHECK(dk <= kScanWaves * 64, "linear_scan: key heads of up to %d channels, not %d", kScanWaves * 64, dk);
   XI_CHECK((z != nullptr) + (head_decay != nullptr) + (step != nullptr) + (gates != nullptr) == 1,
@@ -251,6 +320,7 @@ int xi_linear_scan(const void* q, long long q_stride, const void* k, long long k
   XI_CHECK((in_idx == nullptr || (state_in && in_stride >= (long long)H * dk * dv)) &&
                (out_idx == nullptr || (state_out && out_stride >= (long long)H * dk * dv)),
            "linear_scan: states need a place of at least H dk dv floats each");
+  XI_CHECK(act == 0 || act == 1, "linear_scan: unknown activation %d", act);
   XI_CHECK(first && last, "linear_scan: the items' token ranges are missing");
   if (n_items == 0) return 0;
   dim3 grid((unsigned)n_items, (unsigned)H, (unsigned)((v_cols + kScanCols - 1) / kScanCols));
@@ -260,7 +330,7 @@ int xi_linear_scan(const void* q, long long q_stride, const void* k, long long k
 #define XI_SCAN_ARGS(TT)                                                                                                      \
       (const TT*)q, q_stride, (const TT*)k, k_stride, (const TT*)v, v_stride, z, z_bias, inv_tau, head_decay, (const TT*)step,    \
       step_stride, step_bias, decay_log, gates, v_cols, group_heads, state_in, in_stride,                                                    \
-      in_idx, state_out, out_stride, out_idx, first, last, out, decay_out, H, dk, dv, q_scale, k_scale
+      in_idx, state_out, out_stride, out_idx, first, last, out, decay_out, H, dk, dv, q_scale, k_scale, act
 #define XI_SCAN(TT, R)                                                                                                        \
   do {                                                                                                                        \
     if (z) linear_scan_kernel<TT, R, false><<<grid, kScanWaves * kWave, 0, stream>>>(XI_SCAN_ARGS(TT));                       \
@@ -318,6 +388,31 @@ int xi_head_norm_gate(const float* o, const float* w, float eps, const void* g, 
   else
     XI_CHECK(false, "head_norm_gate: unknown dtype %d", dtype);
   XI_LAUNCH_CHECK("head_norm_gate");
+  return 0;
+}
+
+// o float32 [T, W]; w float32 [W]; g rows of g_stride elements holding [W] gates in `dtype`; act 0: silu, 1: sigmoid;
+// out [T, W] in `dtype`.
+int xi_row_norm_gate(const float* o, const float* w, float eps, const void* g, long long g_stride, int act, void* out, int dtype,
+                     int n_tok, int W, hipStream_t stream) {
+  XI_CHECK(n_tok >= 0 && W > 0 && g_stride >= W && w && (act == 0 || act == 1), "row_norm_gate: bad sizes T=%d W=%d", n_tok, W);
+  XI_CHECK(dtype == kF32 || dtype == kBF16, "row_norm_gate: unknown dtype %d", dtype);
+  if (n_tok == 0) return 0;
+  const uintptr_t run = dtype == kF32 ? 16 : 8;
+  const bool vec = W % 4 == 0 && g_stride % 4 == 0 && reinterpret_cast<uintptr_t>(o) % 16 == 0 && reinterpret_cast<uintptr_t>(w) % 16 == 0 &&
+                   reinterpret_cast<uintptr_t>(g) % run == 0 && reinterpret_cast<uintptr_t>(out) % run == 0;
+#define XI_RNG(TT, NT, VEC) row_norm_gate_kernel<TT, NT, VEC><<<n_tok, NT, 0, stream>>>(o, w, eps, (const TT*)g, g_stride, act, (TT*)out, W)
+#define XI_RNG_T(TT)                                         \
+  do {                                                       \
+    if (!vec) XI_RNG(TT, 256, false);                        \
+    else if (n_tok <= 256 && W > 1024) XI_RNG(TT, 1024, true); \
+    else XI_RNG(TT, 256, true);                              \
+  } while (0)
+  if (dtype == kF32) XI_RNG_T(float);
+  else XI_RNG_T(bf16);
+#undef XI_RNG_T
+#undef XI_RNG
+  XI_LAUNCH_CHECK("row_norm_gate");
   return 0;
 }
 

@@ -2,8 +2,8 @@
 // and the gate and grouped norm behind it.
 //
 // `causal_conv_kernel`: C channels of a packed projection (columns from an offset), each with its own `taps`
-// weights (w [C, taps], w[c, taps - 1 - k] for the input k tokens back) and a bias; out[t, c] = silu(bias[c] + sum_j w[c, j]
-// u[t - (taps - 1) + j, c]), where inputs from before the step's portion are the request's tail (the last taps - 1
+// weights (w [C, taps], w[c, taps - 1 - k] for the input k tokens back) and a bias; out[t, c] = act(bias[c] + sum_j w[c, j]
+// u[t - (taps - 1) + j, c]), act silu or none, where the inputs are u plus a bias of their own (`in_bias`, or none) and inputs from before the step's portion are the request's tail (the last taps - 1
 // inputs of earlier steps, float32 [slots, taps - 1, C], oldest first; zeros for a request's first tokens: a slot
 // is cleared when its request starts).  Sums in float32, one rounding.
 // `conv_tail_kernel` then moves the tail on by the step's tokens (a launch of its own: the tail is read by the
@@ -22,7 +22,8 @@ __global__ __launch_bounds__(256) void causal_conv_kernel(const T* __restrict__ 
                                                           const float* __restrict__ tails, long long slot_stride,
                                                           const long long* __restrict__ slots,
                                                           const int* __restrict__ tok_seq, const int* __restrict__ cu_q,
-                                                          T* __restrict__ out, int C, int taps) {
+                                                          T* __restrict__ out, int C, int taps,
+                                                          const float* __restrict__ in_bias, int act) {
   const int t = blockIdx.x;
   const int c = blockIdx.y * blockDim.x + threadIdx.x;
   if (c >= C) return;
@@ -30,20 +31,21 @@ __global__ __launch_bounds__(256) void causal_conv_kernel(const T* __restrict__ 
   const int t0 = cu_q[b];
   const float* tail = tails + (size_t)slots[b] * slot_stride;
   float acc = bias[c];
+  const float ib = in_bias ? in_bias[c] : 0.f;
   for (int j = 0; j < taps; ++j) {
     const int s = t - (taps - 1) + j;
     // before the portion: s = t0 - k, k = 1 .. taps - 1, the tail's entry taps - 1 - k
-    const float x = s >= t0 ? to_float(u[(size_t)s * u_stride + c]) : tail[(size_t)(taps - 1 - (t0 - s)) * C + c];
+    const float x = s >= t0 ? to_float(u[(size_t)s * u_stride + c]) + ib : tail[(size_t)(taps - 1 - (t0 - s)) * C + c];
     acc = fmaf(w[(size_t)c * taps + j], x, acc);
   }
-  out[(size_t)t * C + c] = from_float<T>(acc / (1.f + expf(-acc)));
+  out[(size_t)t * C + c] = from_float<T>(act ? acc / (1.f + expf(-acc)) : acc);
 }
 
 template <typename T>
 __global__ __launch_bounds__(256) void conv_tail_kernel(const T* __restrict__ u, long long u_stride,
                                                         float* __restrict__ tails, long long slot_stride,
                                                         const long long* __restrict__ slots, const int* __restrict__ cu_q,
-                                                        int C, int taps) {
+                                                        int C, int taps, const float* __restrict__ in_bias) {
   const int b = blockIdx.x;
   const int c = blockIdx.y * blockDim.x + threadIdx.x;
   if (c >= C) return;
@@ -51,11 +53,12 @@ __global__ __launch_bounds__(256) void conv_tail_kernel(const T* __restrict__ u,
   const int n = t1 - t0;
   if (n <= 0) return;
   float* tail = tails + (size_t)slots[b] * slot_stride;
+  const float ib = in_bias ? in_bias[c] : 0.f;
   // entry i of the new tail is the input taps - 1 - i tokens before the end; an entry that is older than the
   // portion is entry i + n of the old tail, which this thread has not overwritten yet (i ascends)
   for (int i = 0; i < taps - 1; ++i) {
     const int s = t1 - (taps - 1) + i;
-    tail[(size_t)i * C + c] = s >= t0 ? to_float(u[(size_t)s * u_stride + c]) : tail[(size_t)(i + n) * C + c];
+    tail[(size_t)i * C + c] = s >= t0 ? to_float(u[(size_t)s * u_stride + c]) + ib : tail[(size_t)(i + n) * C + c];
   }
 }
 
@@ -124,15 +127,17 @@ __global__ __launch_bounds__(256) void causal_conv_run_kernel(const T* __restric
                                                               const float* __restrict__ tails, long long slot_stride,
                                                               const long long* __restrict__ slots,
                                                               const int* __restrict__ tok_seq, const int* __restrict__ cu_q,
-                                                              T* __restrict__ out, int n_tok, int C, int run) {
+                                                              T* __restrict__ out, int n_tok, int C, int run,
+                                                              const float* __restrict__ in_bias, int act) {
   const int c = 8 * (blockIdx.y * blockDim.x + threadIdx.x);
   if (c >= C) return;
   const int ta = blockIdx.x * run;
   const int tb = ta + run < n_tok ? ta + run : n_tok;
-  float wt[TAPS][8], bs[8], win[TAPS > 1 ? TAPS - 1 : 1][8];
+  float wt[TAPS][8], bs[8], ib[8], win[TAPS > 1 ? TAPS - 1 : 1][8];
 #pragma unroll
   for (int i = 0; i < 8; ++i) {
     bs[i] = bias[c + i];
+    ib[i] = in_bias ? in_bias[c + i] : 0.f;
 #pragma unroll
     for (int j = 0; j < TAPS; ++j) wt[j][i] = w[(size_t)(c + i) * TAPS + j];
   }
@@ -146,19 +151,25 @@ __global__ __launch_bounds__(256) void causal_conv_run_kernel(const T* __restric
 #pragma unroll
       for (int i = 0; i < TAPS - 1; ++i) {
         const int s = t - (TAPS - 1) + i;
-        if (s >= t0) load8(u + (size_t)s * u_stride + c, win[i]);
-        else load8(tail + (size_t)(TAPS - 1 - (t0 - s)) * C + c, win[i]);
+        if (s >= t0) {
+          load8(u + (size_t)s * u_stride + c, win[i]);
+#pragma unroll
+          for (int e = 0; e < 8; ++e) win[i][e] += ib[e];
+        } else {
+          load8(tail + (size_t)(TAPS - 1 - (t0 - s)) * C + c, win[i]);      // (kept with their bias)
+        }
       }
     }
     float cur[8], o[8];
     load8(u + (size_t)t * u_stride + c, cur);
 #pragma unroll
     for (int i = 0; i < 8; ++i) {
+      cur[i] += ib[i];
       float acc = bs[i];
 #pragma unroll
       for (int j = 0; j < TAPS - 1; ++j) acc = fmaf(wt[j][i], win[j][i], acc);
       acc = fmaf(wt[TAPS - 1][i], cur[i], acc);
-      o[i] = acc / (1.f + expf(-acc));
+      o[i] = act ? acc / (1.f + expf(-acc)) : acc;
     }
     store8(out + (size_t)t * C + c, o);
 #pragma unroll
@@ -241,10 +252,10 @@ extern "C" {
 
 // u: rows of u_stride elements whose first C (from the given pointer) are the channels; w float32 [C, taps], bias
 // float32 [C]; tails float32, slot s at tails + s * slot_stride, [taps - 1, C] each; slots int64 [B]; tok_seq int32 [T];
-// cu_q int32 [B + 1]; out [T, C] in `dtype`.
+// cu_q int32 [B + 1]; out [T, C] in `dtype`; in_bias float32 [C] or null, added to u (the tails hold it already); act 1: silu, 0: none.
 int xi_causal_conv(const void* u, long long u_stride, int dtype, const float* w, const float* bias, const float* tails,
                    long long slot_stride, const long long* slots, const int* tok_seq, const int* cu_q, void* out, int n_tok,
-                   int C, int taps, hipStream_t stream) {
+                   int C, int taps, const float* in_bias, int act, hipStream_t stream) {
   XI_CHECK(n_tok >= 0 && C > 0 && taps >= 1 && u_stride >= C, "causal_conv: bad sizes T=%d C=%d taps=%d", n_tok, C, taps);
   XI_CHECK(slot_stride >= (long long)(taps - 1) * C, "causal_conv: a slot's tail is too small");
   if (n_tok == 0) return 0;
@@ -257,7 +268,7 @@ int xi_causal_conv(const void* u, long long u_stride, int dtype, const float* w,
     dim3 vgrid((unsigned)((n_tok + run - 1) / run), (unsigned)((C / 8 + 255) / 256));
 #define XI_CONV_RUN(TT, TAPS)                                                                                          \
   causal_conv_run_kernel<TT, TAPS><<<vgrid, 256, 0, stream>>>((const TT*)u, u_stride, w, bias, tails, slot_stride, slots, \
-                                                             tok_seq, cu_q, (TT*)out, n_tok, C, run)
+                                                             tok_seq, cu_q, (TT*)out, n_tok, C, run, in_bias, act)
 #define XI_CONV_TAPS(TT)              \
   switch (taps) {                     \
     case 1: XI_CONV_RUN(TT, 1); break; \
@@ -280,10 +291,10 @@ int xi_causal_conv(const void* u, long long u_stride, int dtype, const float* w,
   XI_CHECK(grid.y <= 65535u, "causal_conv: too many channels");
   if (dtype == kF32)
     causal_conv_kernel<float><<<grid, 256, 0, stream>>>((const float*)u, u_stride, w, bias, tails, slot_stride, slots, tok_seq,
-                                                        cu_q, (float*)out, C, taps);
+                                                        cu_q, (float*)out, C, taps, in_bias, act);
   else if (dtype == kBF16)
     causal_conv_kernel<bf16><<<grid, 256, 0, stream>>>((const bf16*)u, u_stride, w, bias, tails, slot_stride, slots, tok_seq,
-                                                       cu_q, (bf16*)out, C, taps);
+                                                       cu_q, (bf16*)out, C, taps, in_bias, act);
   else
     XI_CHECK(false, "causal_conv: unknown dtype %d", dtype);
   XI_LAUNCH_CHECK("causal_conv");
@@ -291,16 +302,16 @@ int xi_causal_conv(const void* u, long long u_stride, int dtype, const float* w,
 }
 
 int xi_conv_tail(const void* u, long long u_stride, int dtype, float* tails, long long slot_stride, const long long* slots,
-                 const int* cu_q, int n_seqs, int C, int taps, hipStream_t stream) {
+                 const int* cu_q, int n_seqs, int C, int taps, const float* in_bias, hipStream_t stream) {
   XI_CHECK(n_seqs >= 0 && C > 0 && taps >= 1 && u_stride >= C, "conv_tail: bad sizes B=%d C=%d taps=%d", n_seqs, C, taps);
   XI_CHECK(slot_stride >= (long long)(taps - 1) * C, "conv_tail: a slot's tail is too small");
   if (n_seqs == 0 || taps == 1) return 0;
   dim3 grid((unsigned)n_seqs, (unsigned)((C + 255) / 256));
   XI_CHECK(grid.y <= 65535u, "conv_tail: too many channels");
   if (dtype == kF32)
-    conv_tail_kernel<float><<<grid, 256, 0, stream>>>((const float*)u, u_stride, tails, slot_stride, slots, cu_q, C, taps);
+    conv_tail_kernel<float><<<grid, 256, 0, stream>>>((const float*)u, u_stride, tails, slot_stride, slots, cu_q, C, taps, in_bias);
   else if (dtype == kBF16)
-    conv_tail_kernel<bf16><<<grid, 256, 0, stream>>>((const bf16*)u, u_stride, tails, slot_stride, slots, cu_q, C, taps);
+    conv_tail_kernel<bf16><<<grid, 256, 0, stream>>>((const bf16*)u, u_stride, tails, slot_stride, slots, cu_q, C, taps, in_bias);
   else
     XI_CHECK(false, "conv_tail: unknown dtype %d", dtype);
   XI_LAUNCH_CHECK("conv_tail");

@@ -19,6 +19,7 @@ from ..parts import (KVNeed, LayerCache, StateNeed, StepContext, Stream, block_c
                      head_class, norm_class, state_needs_of, stream_op_class)
 
 EMBEDDING_CACHE = -1        # the key of the state that the embedding keeps (no layer's index, no run's cache id)
+from ..parts.joining import closed, join, joins
 from ..weights.store import TensorDecl, WeightStore
 
 
@@ -39,12 +40,15 @@ class CausalLM:
         self.blocks = [block_class(l.block)(l, dtype) for l in spec.layers]
         self.final_norm = norm_class(spec.final_norm.kind)(spec.final_norm, dtype)
         self.head = head_class(spec.head.kind)(spec.head, dtype)
-        # what runs on the stream before a schedule entry's layer: one object a distinct spec
+        # what runs on the stream before or after a schedule entry's layer: one object a distinct spec
         self.stream_ops = {}
         for e in spec.schedule:
-            if e.before is not None and id(e.before) not in self.stream_ops:
-                self.stream_ops[id(e.before)] = stream_op_class(e.before.kind)(e.before, dtype)
+            for op in self._ops_of(e):
+                if id(op) not in self.stream_ops:
+                    self.stream_ops[id(op)] = stream_op_class(op.kind)(op, dtype)
         self._keep_first = any(op.needs_first for op in self.stream_ops.values())
+        # the embedding's output is kept as a copy only if something changes the stream's tensor in place
+        self._copy_first = any(p.writes_stream for p in (*self.blocks, *self.stream_ops.values()))
         for e in spec.schedule:
             if not (0 <= e.layer < len(self.blocks)):
                 raise ValueError(f"schedule names layer {e.layer} but the model has {len(self.blocks)}")
@@ -61,6 +65,10 @@ class CausalLM:
         """Every part can be recorded into a HIP graph (see `Part.graph_safe`)."""
         return all(p.graph_safe for p in (self.embedding, self.final_norm, self.head, *self.blocks, *self.stream_ops.values()))
 
+    @staticmethod
+    def _ops_of(e):
+        return (() if e.before is None else (e.before,)) + tuple(e.after)
+
     # ---- weights -------------------------------------------------------------
     @classmethod
     def declare(cls, spec: ModelSpec) -> List[TensorDecl]:
@@ -68,8 +76,8 @@ class CausalLM:
         for l in spec.layers:
             decls += block_class(l.block).declare(l)
         for e in spec.schedule:
-            if e.before is not None:
-                decls += stream_op_class(e.before.kind).declare(e.before, "")
+            for op in CausalLM._ops_of(e):
+                decls += stream_op_class(op.kind).declare(op, "")
         decls += norm_class(spec.final_norm.kind).declare(spec.final_norm, str(spec.final_norm.get("prefix", "")))
         decls += head_class(spec.head.kind).declare(spec.head)
         seen, out = set(), []
@@ -147,11 +155,17 @@ class CausalLM:
                 want_rows: torch.Tensor) -> torch.Tensor:
         """ids int32 [T]; caches: layer index -> the cache that layer owns; want_rows int32
         [R].  Returns float32 logits [R, vocab]."""
+        ctx.ids = ids
         if EMBEDDING_CACHE in self.state_needs:
             first = self.embedding.forward(ids, ctx, cache=caches[EMBEDDING_CACHE])
         else:
             first = self.embedding.forward(ids, ctx)
-        kept_first = first.clone() if self._keep_first else None       # the norms add into `first` in place
+        kept_first = None
+        if self._keep_first:             # most norms add into `first` in place
+            kept_first = first.clone() if self._copy_first else first
+
+        def run_op(op, stream):
+            return op.forward(stream if op.takes_open else closed(stream), kept_first, ctx)
         # an embedding kind may also hand on its result rounded to the activation dtype (`rows`)
         stream = Stream(first, None, rows=getattr(self.embedding, "rows", None))
         schedule = self.spec.schedule
@@ -162,17 +176,25 @@ class CausalLM:
             elif e.cache_of is not None:
                 c = LayerCache(c.group, c.pools, c.state, write=False, states=c.states)
             if e.before is not None:
-                stream = self.stream_ops[id(e.before)].forward(stream, kept_first, ctx)
+                stream = run_op(self.stream_ops[id(e.before)], stream)
             blk = self.blocks[e.layer]
+            if stream.open and not blk.takes_open:
+                stream = closed(stream)
             if getattr(blk, "folds", False):
                 # the block that runs next may let this one half do its first norm
                 nxt = self.blocks[schedule[i + 1].layer] if i + 1 < len(schedule) else None
                 next_norm = nxt.first_norm() if getattr(nxt, "folds", False) else None
-                if nxt is not None and schedule[i + 1].before is not None:
+                if e.after or (nxt is not None and schedule[i + 1].before is not None):
                     next_norm = None          # something changes the stream in between: the norm sees another sum
                 stream = blk.forward(stream, ctx, c, next_norm=next_norm)
             else:
                 stream = blk.forward(stream, ctx, c)
+            for op in e.after:
+                stream = run_op(self.stream_ops[id(op)], stream)
+        if stream.open and joins(self.final_norm):
+            h = join(stream, self.dtype, (self.final_norm,), rows=want_rows)[2][0]
+            return self.head.forward(h)
+        stream = closed(stream)
         if stream.pending is not None and stream.pending_scale != 1.0:
             h = self.final_norm.forward(stream.resid, stream.pending, self.dtype, rows=want_rows,
                                         add_scale=stream.pending_scale)

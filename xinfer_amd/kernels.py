@@ -277,7 +277,7 @@ def scan_chunk_plan(q_lens, chunk: Optional[int] = None):
     return whole, long, chunks
 
 
-def _scan_launch(q, k, v, qs, ks, vs, z, z_bias, tau, head_decay, step, ss, step_bias, decay_log, gates, v_cols, group_heads,
+def _scan_launch(q, k, v, qs, ks, vs, z, z_bias, tau, head_decay, step, ss, step_bias, decay_log, gates, v_cols, group_heads, act,
                  state_in, in_stride, in_idx, state_out, out_stride, out_idx,
                  first, last, out, decay_out, items, H, dk, dv, q_scale, k_scale):
     _ok(lib().xi_linear_scan(_p(q), ctypes.c_longlong(qs), _p(k), ctypes.c_longlong(ks), _p(v), ctypes.c_longlong(vs),
@@ -286,7 +286,7 @@ def _scan_launch(q, k, v, qs, ks, vs, z, z_bias, tau, head_decay, step, ss, step
                              int(group_heads), _p(state_in),
                              ctypes.c_longlong(in_stride), _p(in_idx), _p(state_out), ctypes.c_longlong(out_stride),
                              _p(out_idx), ctypes.c_void_p(first), ctypes.c_void_p(last), _p(out), _p(decay_out), int(items),
-                             H, dk, dv, ctypes.c_float(q_scale), ctypes.c_float(k_scale), _stream()))
+                             H, dk, dv, ctypes.c_float(q_scale), ctypes.c_float(k_scale), int(act), _stream()))
 
 
 def linear_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: torch.Tensor, state_slots: torch.Tensor,
@@ -295,7 +295,7 @@ def linear_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: torch.
                 k_scale: float = 1.0, z_bias: Optional[torch.Tensor] = None, q_lens=None, plan_cache=None,
                 step: Optional[torch.Tensor] = None, step_bias: Optional[torch.Tensor] = None,
                 decay_log: Optional[torch.Tensor] = None, groups: Optional[int] = None,
-                gates: Optional[torch.Tensor] = None, value_cols: Optional[int] = None) -> torch.Tensor:
+                gates: Optional[torch.Tensor] = None, value_cols: Optional[int] = None, silu: bool = False) -> torch.Tensor:
     """Linear attention with a decaying float32 state per request and head, S <- diag(a) S + k v^T, o = S^T q,
     token by token from the state each request's slot holds (left there afterwards).  q, k [T, H dk] and
     v [T, H dv] may be column ranges of a packed projection.  The decay: `z` float32 [T, H dk], `z_bias`
@@ -305,6 +305,7 @@ def linear_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: torch.
     Or `gates` float32 [T, H, 2], made beforehand: a = gates[t, h, 0] and the token's value row times gates[t, h, 1].
     `value_cols` = value_dim - 1: v is [T, H (value_dim - 1)] and the state's last column reads the value 1 (it then
     holds the decayed sum of the weighted keys alone, and the results' last column that sum times q).
+    `silu`: q, k and v pass silu first (in float32, before any factor).
     `groups` G: q and k are [T, G dk] and head h reads the columns of group h // (H / G).
     state float32 [slots, H, dk, dv] (slots may be strided); state_slots int64 [B]; cu_q int32 [B + 1].
     Returns o float32 [T, H, dv].
@@ -369,7 +370,7 @@ def linear_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: torch.
         raise KernelError("linear_scan: the portions' lengths do not add up to the step's tokens")
     out = torch.empty((T, H, dv), dtype=torch.float32, device=q.device)
     slot_stride = int(state.stride(0)) if state.shape[0] > 1 else H * dk * dv
-    common = (q, k, v, qs, ks, vs, z, z_bias, tau, head_decay, step, ss, step_bias, decay_log, gates, vc, H // G)
+    common = (q, k, v, qs, ks, vs, z, z_bias, tau, head_decay, step, ss, step_bias, decay_log, gates, vc, H // G, int(bool(silu)))
     whole, long, chunks = scan_chunk_plan(q_lens) if q_lens is not None else (None, [], [])
     if not long:            # every request in one piece, straight from the step's own arrays
         _scan_launch(*common, state, slot_stride, state_slots, state, slot_stride, state_slots, cu_q.data_ptr(),
@@ -803,12 +804,13 @@ def attention_generic(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Ten
                       scale: float, window: int = 0, out: Optional[torch.Tensor] = None,
                       v_grouped: bool = False, softcap: float = 0.0,
                       slopes: Optional[torch.Tensor] = None, sinks: Optional[torch.Tensor] = None,
-                      value_dim: Optional[int] = None) -> torch.Tensor:
+                      value_dim: Optional[int] = None, chunk: int = 0) -> torch.Tensor:
     """Causal paged GQA attention for any mix of tokens.  q [T, nq, d]; caches
     [pages, nkv, page_size, d] (the V pool's last size, the value head size, may differ);
     block_tables int32 [B, max_pages]; tok_seq / positions
     int32 [T] name each token's row of block_tables and its absolute position.
-    window = 0 keeps all keys, w > 0 the last w (the query's own key included).
+    window = 0 keeps all keys, w > 0 the last w (the query's own key included); chunk c > 0 keeps the keys of the query's
+    own chunk of c positions (counted from position 0).
     `softcap` c > 0: scores become c * tanh(score / c); `slopes` float32 [nq]: head h's scores lose
     slopes[h] * (distance from the query to the key); `sinks` float32 [nq]: head h's softmax has exp(sinks[h]) in
     its denominator beside the keys' weights.  `v_cache` None: a key's first `value_dim` dims are its value (one
@@ -852,7 +854,7 @@ def attention_generic(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Ten
         _p(q), _p(k_cache), _p(v_cache), _code(q, "attention"), _p(block_tables),
         int(block_tables.shape[1]), _p(tok_seq), _p(positions), _p(out), ctypes.c_float(scale),
         int(window), int(page), T, nq, nkv, d, dv, int(bool(v_grouped)), ctypes.c_float(softcap), _p(slopes), _p(sinks),
-        int(v_cache is None), nkk, _stream()))
+        int(v_cache is None), nkk, int(chunk), _stream()))
     return out
 
 
@@ -1074,9 +1076,9 @@ def biased_split_keys(workgroups: int, span: int) -> int:
 
 
 def attention_biased_bf16(q, k_cache, vt_cache, block_tables, tiles, cu_q, ctx_lens, scale, window=0, softcap=0.0,
-                          slopes=None, out=None, small=0, split_keys=0, span=0, sinks=None, rows_heads=0):
+                          slopes=None, out=None, small=0, split_keys=0, span=0, sinks=None, rows_heads=0, chunk=0):
     """Matrix-core attention for any mix of portions with the score's options (`softcap`, `slopes`: see
-    `attention_generic`; `sinks` as there) and a value head size of its own: q [T, nq, d], K pool [pages, nkv, page, d], V pool
+    `attention_generic`; `sinks` and `chunk` as there) and a value head size of its own: q [T, nq, d], K pool [pages, nkv, page, d], V pool
     [pages, nkv, page / 8, dv, 8]; tiles int32 [n, 2] = (sequence, first query token of a block of
     `attention_biased_block(d, dv, nq // nkv, small)` tokens within the sequence's portion).  Returns [T, nq * dv].
     `split_keys` > 0 (steps in which every sequence brings one token, a tile a token): each workgroup walks one slice
@@ -1133,7 +1135,7 @@ def attention_biased_bf16(q, k_cache, vt_cache, block_tables, tiles, cu_q, ctx_l
         _p(q), _p(k_cache), _p(vt_cache), _p(block_tables), int(block_tables.shape[1]), _p(tiles), int(tiles.shape[0]),
         _p(cu_q), _p(ctx_lens), _p(out), ctypes.c_float(scale), ctypes.c_float(softcap), _p(slopes), _p(sinks), int(window),
         int(page), nq, nkv, d, dv, int(small), _p(part_o), _p(part_ml), int(split_keys), int(max_splits), int(T), int(rows_heads),
-        nkk, rows_kv, _stream()))
+        nkk, rows_kv, int(chunk), _stream()))
     return out
 
 
@@ -1225,12 +1227,12 @@ def attention_decode_packed_bf16(qkv, q_weight, k_weight, eps, cos, sin, rotary_
 def attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, ctx, group: int,
               scale: float, window: int = 0, v_grouped: bool = False, softcap: float = 0.0,
               slopes: Optional[torch.Tensor] = None, sinks: Optional[torch.Tensor] = None,
-              value_dim: Optional[int] = None) -> torch.Tensor:
+              value_dim: Optional[int] = None, chunk: int = 0) -> torch.Tensor:
     """Attention of one step's tokens over the paged cache of `group`; chooses the kernel
     from the precision and the shape of the batch: float32, or sizes the matrix-core
     kernels do not take, go to the generic kernel; bfloat16 batches of single tokens to
     the split-K decode kernel; everything else to the prefill kernel.  Scores with a soft cap
-    or a distance bias, a softmax with sinks, and values of another head size than the keys, have
+    or a distance bias, a softmax with sinks, keys seen by chunks, and values of another head size than the keys, have
     matrix-core kernels of their own (`attention_biased_bf16`).  `v_cache` None: a key's first
     `value_dim` dims are its value, which only the generic kernel reads that way."""
     T, nq, d = q.shape
@@ -1239,9 +1241,11 @@ def attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, ctx
     bt = ctx.block_tables[group]
     if v_cache is None:
         return attention_generic(q, k_cache, None, bt, ctx.tok_seq, ctx.positions, scale, window, softcap=softcap,
-                                 slopes=slopes, sinks=sinks, value_dim=value_dim)
-    if softcap > 0 or slopes is not None or sinks is not None or v_cache.shape[3] != d or nkk != nkv:
+                                 slopes=slopes, sinks=sinks, value_dim=value_dim, chunk=chunk)
+    if chunk > 0 or softcap > 0 or slopes is not None or sinks is not None or v_cache.shape[3] != d or nkk != nkv:
         dv = int(v_cache.shape[3])
+        # the most keys a single token sees, and up to a tile before them
+        seen = min([n for n in (int(window), int(chunk)) if n > 0], default=0)
         if q.dtype == torch.bfloat16 and v_grouped and BIASED_MFMA and attention_biased_supported(nq, nkv, d, dv, page):
             if (ctx.max_q_len == 1 and nkk == 1 and nkv > 1 and nq // nkv >= HEAD_ROWS_FROM and slopes is None and sinks is None
                     and q.is_contiguous()):
@@ -1263,10 +1267,10 @@ def attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, ctx
                     cached = (torch.stack([seqs, first], dim=1).contiguous(), small, ctx.cu_q * nq, blocks)
                     ctx.scratch[key] = cached
                 tiles, small, cu_rows, blocks = cached
-                span = min(int(ctx.max_ctx_len), int(window) + 63) if window > 0 else int(ctx.max_ctx_len)
+                span = min(int(ctx.max_ctx_len), seen + 63) if seen else int(ctx.max_ctx_len)
                 split = biased_split_keys(ctx.num_seqs * blocks, span)
                 out = attention_biased_bf16(q.view(T * nq, 1, d), k_cache, v_cache, bt, tiles, cu_rows, ctx.ctx_lens, scale, window,
-                                            softcap=softcap, small=small, split_keys=split, span=span, rows_heads=nq)
+                                            softcap=softcap, small=small, split_keys=split, span=span, rows_heads=nq, chunk=chunk)
                 return out.view(T, nq * dv)
             if ctx.max_q_len == 1 and nkv == 1 and nq >= HEAD_ROWS_FROM and slopes is None and q.is_contiguous():
                 # single tokens whose heads all read the one kv head: the heads are the rows of a block, so a tile
@@ -1282,10 +1286,10 @@ def attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, ctx
                     cached = (torch.stack([seqs, first], dim=1).contiguous(), small, ctx.cu_q * nq, blocks)
                     ctx.scratch[key] = cached
                 tiles, small, cu_rows, blocks = cached
-                span = min(int(ctx.max_ctx_len), int(window) + 63) if window > 0 else int(ctx.max_ctx_len)
+                span = min(int(ctx.max_ctx_len), seen + 63) if seen else int(ctx.max_ctx_len)
                 split = biased_split_keys(ctx.num_seqs * blocks, span)
                 out = attention_biased_bf16(q.view(T * nq, 1, d), k_cache, v_cache, bt, tiles, cu_rows, ctx.ctx_lens, scale, window,
-                                            softcap=softcap, small=small, split_keys=split, span=span, sinks=sinks, rows_heads=nq)
+                                            softcap=softcap, small=small, split_keys=split, span=span, sinks=sinks, rows_heads=nq, chunk=chunk)
                 return out.view(T, nq * dv)
             key = ("attention_biased_tiles", d, dv, nq, nkv)
             cached = ctx.scratch.get(key)
@@ -1303,12 +1307,12 @@ def attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, ctx
             split, span = 0, 0
             if ctx.max_q_len == 1:           # single tokens: slices of the keys where the sequences alone leave the chip idle
                 g = nq // nkv
-                span = min(int(ctx.max_ctx_len), int(window) + 63) if window > 0 else int(ctx.max_ctx_len)
+                span = min(int(ctx.max_ctx_len), seen + 63) if seen else int(ctx.max_ctx_len)
                 split = biased_split_keys(ctx.num_seqs * nkv * (g // (4 if g % 4 == 0 else 2 if g % 2 == 0 else 1)), span)
             return attention_biased_bf16(q, k_cache, v_cache, bt, tiles, ctx.cu_q, ctx.ctx_lens, scale, window,
-                                         softcap=softcap, slopes=slopes, small=small, split_keys=split, span=span, sinks=sinks)
+                                         softcap=softcap, slopes=slopes, small=small, split_keys=split, span=span, sinks=sinks, chunk=chunk)
         return attention_generic(q, k_cache, v_cache, bt, ctx.tok_seq, ctx.positions, scale, window,
-                                 v_grouped=v_grouped, softcap=softcap, slopes=slopes, sinks=sinks)
+                                 v_grouped=v_grouped, softcap=softcap, slopes=slopes, sinks=sinks, chunk=chunk)
     if q.dtype == torch.bfloat16 and v_grouped and mfma_attention_supported(nq, nkv, d, page):
         g = nq // nkv
         if ctx.max_q_len == 1 and decode_attention_takes(nq, nkv, d):
@@ -1799,12 +1803,15 @@ def stream_start(resid: torch.Tensor, pending: Optional[torch.Tensor], factor: f
 def head_rows(qkv: torch.Tensor, slots: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, num_heads: int,
               num_kv_heads: int, head_dim: int, value_dim: int, v_grouped: bool = False, cos: Optional[torch.Tensor] = None,
               sin: Optional[torch.Tensor] = None, rotary_dim: int = 0, interleaved: bool = False,
-              positions: Optional[torch.Tensor] = None, unit_norm: bool = False, eps: float = 0.0) -> torch.Tensor:
-    """A packed projection [T, nq d + nkv d + nkv dv]: the first `rotary_dim` dims of every q and k head turn by the
+              positions: Optional[torch.Tensor] = None, unit_norm: bool = False, eps: float = 0.0,
+              bias: Optional[torch.Tensor] = None, q_weight: Optional[torch.Tensor] = None,
+              k_weight: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """A packed projection [T, nq d + nkv d + nkv dv]: `bias` (float32, one number a column) is added, every q and k head
+    is divided by its root mean square over d and multiplied by `q_weight` / `k_weight` (float32 [d]; none: not), the first `rotary_dim` dims of every q and k head turn by the
     token's position (pairs (2i, 2i + 1) if `interleaved`, else (i, i + r / 2); `cos` / `sin` float32 [positions, r / 2]),
     then, with `unit_norm`, each head is divided by its root mean square over d (eps inside the root); k and v go into
     the paged cache at `slots`.  Returns q [T, nq, d]."""
-    _dev(qkv, slots, k_cache, v_cache, cos, sin, positions)
+    _dev(qkv, slots, k_cache, v_cache, cos, sin, positions, bias, q_weight, k_weight)
     nq, nkv, d, dv, rot = int(num_heads), int(num_kv_heads), int(head_dim), int(value_dim), int(rotary_dim)
     if qkv.dim() != 2 or qkv.shape[1] != nq * d + nkv * d + nkv * dv:
         raise KernelError(f"head_rows: qkv {tuple(qkv.shape)} is not [T, {nq * d + nkv * d + nkv * dv}]")
@@ -1821,11 +1828,18 @@ def head_rows(qkv: torch.Tensor, slots: torch.Tensor, k_cache: torch.Tensor, v_c
         if cos.shape != sin.shape or cos.dim() != 2 or cos.shape[1] != rot // 2 or positions.shape != (T,):
             raise KernelError(f"head_rows: the rotation's tables must be [positions, {rot // 2}], positions [T]")
     _check_cache(k_cache, v_cache, nkv, d, qkv.dtype, v_grouped, "head_rows", dv=dv)
+    if (q_weight is None) != (k_weight is None):
+        raise KernelError("head_rows: q and k norm weights come together")
+    for w, n in ((bias, qkv.shape[1]), (q_weight, d), (k_weight, d)):
+        if w is not None:
+            _want(w, torch.float32, "head_rows: bias and norm weights")
+            if w.shape != (n,):
+                raise KernelError(f"head_rows: a bias or weight of {tuple(w.shape)} is not [{n}]")
     q_out = torch.empty((T, nq, d), dtype=qkv.dtype, device=qkv.device)
     _ok(lib().xi_head_rows(_p(qkv), _code(qkv, "head_rows"), _p(slots), _p(q_out), _p(k_cache), _p(v_cache),
                            int(k_cache.shape[2]), T, nq, nkv, d, dv, int(bool(v_grouped)), _p(cos if rot else None),
                            _p(sin if rot else None), rot, int(bool(interleaved)), _p(positions if rot else None),
-                           int(bool(unit_norm)), ctypes.c_float(eps), _stream()))
+                           int(bool(unit_norm)), ctypes.c_float(eps), _p(bias), _p(q_weight), _p(k_weight), _stream()))
     return q_out
 
 
@@ -1873,10 +1887,11 @@ def head_linear(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor, gate: Optio
     """out[t, h, n] = sum_k x[t, h, k] * w[h, n, k] for every head, float32 sums; with `gate`
     [T, H, N], out *= sigmoid(gate); a gate [T, H] is one number a head.  bfloat16 operands whose K is contiguous in whole 16-byte chunks run on the
     matrix cores; others, and float32, on the vector units in ascending k.  All operands may be strided views ([T, H, .] of packed rows; w [H, N, K] with
-    either N or K contiguous) of one type; `out` [T, H, N] is written in place."""
+    either N or K contiguous) of one type; `out` [T, H, N] is written in place (in that type, or float32: then on the vector units)."""
     for t in (x, w, out, gate):
-        if t is not None and (not t.is_cuda or t.dtype != x.dtype or t.device != x.device):
-            raise KernelError("head_linear: operands of one type on one GPU")
+        if t is not None and (not t.is_cuda or t.device != x.device
+                              or (t.dtype != x.dtype and not (t is out and t.dtype == torch.float32))):
+            raise KernelError("head_linear: operands of one type on one GPU (results in that type or float32)")
     if x.dim() != 3 or w.dim() != 3 or out.dim() != 3:
         raise KernelError("head_linear: x [T, H, K], w [H, N, K], out [T, H, N]")
     T, H, K = x.shape
@@ -1891,18 +1906,26 @@ def head_linear(x: torch.Tensor, w: torch.Tensor, out: torch.Tensor, gate: Optio
     g = gate if gate is not None else out
     _ok(lib().xi_head_linear(_p(x), ll(x.stride(0)), ll(x.stride(1)), _p(w), ll(w.stride(0)), ll(w.stride(1)), ll(w.stride(2)),
                              _p(out), ll(out.stride(0)), ll(out.stride(1)), _p(gate), ll(g.stride(0)), ll(g.stride(1)),
-                             int(each), _code(x, "head_linear"), T, H, N, K, _stream()))
+                             int(each), _code(x, "head_linear"), _code(out, "head_linear"), T, H, N, K, _stream()))
     return out
 
 
 # ---- around the state of a selective state-space mixer ---------------------------------------------------------
+def _conv_in_bias(in_bias: Optional[torch.Tensor], C: int, what: str) -> None:
+    if in_bias is not None:
+        _want(in_bias, torch.float32, f"{what}: in_bias")
+        if in_bias.shape != (C,):
+            raise KernelError(f"{what}: the inputs' bias {tuple(in_bias.shape)} is not [{C}]")
+
+
 def causal_conv(u: torch.Tensor, weight: torch.Tensor, bias: torch.Tensor, tails: torch.Tensor, state_slots: torch.Tensor,
-                tok_seq: torch.Tensor, cu_q: torch.Tensor) -> torch.Tensor:
-    """out[t, c] = silu(bias[c] + sum_j weight[c, j] u[t - (taps - 1) + j, c]) within each sequence; inputs from before
+                tok_seq: torch.Tensor, cu_q: torch.Tensor, in_bias: Optional[torch.Tensor] = None, act: str = "silu") -> torch.Tensor:
+    """out[t, c] = act(bias[c] + sum_j weight[c, j] u[t - (taps - 1) + j, c]) within each sequence, act "silu" or "none", u with
+    `in_bias` (float32 [C]; none: nothing) added; inputs from before
     the step's portion come from the request's tail (`tails` float32 [slots, taps - 1, C], oldest first; slots may be
     strided), which is left as it is (`conv_tail` moves it on).  u [T, C] may be columns of a packed projection;
     weight float32 [C, taps], bias float32 [C].  Returns [T, C] in u's type."""
-    _dev(weight, bias, state_slots, tok_seq, cu_q)
+    _dev(weight, bias, state_slots, tok_seq, cu_q, in_bias)
     T, C = u.shape
     us = _columns(u, C, "causal_conv: u")
     _want(weight, torch.float32, "causal_conv: weight")
@@ -1918,16 +1941,22 @@ def causal_conv(u: torch.Tensor, weight: torch.Tensor, bias: torch.Tensor, tails
     if (tails.dim() != 3 or tuple(tails.shape[1:]) != (taps - 1, C) or not tails.is_cuda or tails.device != u.device
             or (taps > 1 and tails[0].stride() != (C, 1))):
         raise KernelError(f"causal_conv: tails {tuple(tails.shape)} must be [slots, {taps - 1}, {C}] with whole slots")
+    _conv_in_bias(in_bias, C, "causal_conv")
+    if act not in ("silu", "none"):
+        raise KernelError(f"causal_conv: unknown activation {act!r}")
     out = torch.empty((T, C), dtype=u.dtype, device=u.device)
     stride = int(tails.stride(0)) if tails.shape[0] > 1 else (taps - 1) * C
     _ok(lib().xi_causal_conv(_p(u), ctypes.c_longlong(us), _code(u, "causal_conv"), _p(weight), _p(bias), _p(tails),
-                             ctypes.c_longlong(stride), _p(state_slots), _p(tok_seq), _p(cu_q), _p(out), T, C, taps, _stream()))
+                             ctypes.c_longlong(stride), _p(state_slots), _p(tok_seq), _p(cu_q), _p(out), T, C, taps, _p(in_bias),
+                             int(act == "silu"), _stream()))
     return out
 
 
-def conv_tail(u: torch.Tensor, tails: torch.Tensor, state_slots: torch.Tensor, cu_q: torch.Tensor) -> None:
-    """Moves every request's tail on by its portion of this step: afterwards it holds the last taps - 1 inputs."""
-    _dev(state_slots, cu_q)
+def conv_tail(u: torch.Tensor, tails: torch.Tensor, state_slots: torch.Tensor, cu_q: torch.Tensor,
+              in_bias: Optional[torch.Tensor] = None) -> None:
+    """Moves every request's tail on by its portion of this step: afterwards it holds the last taps - 1 inputs (with
+    `in_bias` added, see `causal_conv`)."""
+    _dev(state_slots, cu_q, in_bias)
     T, C = u.shape
     us = _columns(u, C, "conv_tail: u")
     _want(tails, torch.float32, "conv_tail: tails")
@@ -1936,12 +1965,13 @@ def conv_tail(u: torch.Tensor, tails: torch.Tensor, state_slots: torch.Tensor, c
     B = state_slots.shape[0]
     if tails.dim() != 3 or tails.shape[2] != C or cu_q.shape != (B + 1,) or not tails.is_cuda or tails.device != u.device:
         raise KernelError(f"conv_tail: tails {tuple(tails.shape)} must be [slots, taps - 1, {C}], cu_q [B + 1]")
+    _conv_in_bias(in_bias, C, "conv_tail")
     taps = int(tails.shape[1]) + 1
     if taps > 1 and tails[0].stride() != (C, 1):
         raise KernelError("conv_tail: whole slots")
     stride = int(tails.stride(0)) if tails.shape[0] > 1 else (taps - 1) * C
     _ok(lib().xi_conv_tail(_p(u), ctypes.c_longlong(us), _code(u, "conv_tail"), _p(tails), ctypes.c_longlong(stride),
-                           _p(state_slots), _p(cu_q), B, C, taps, _stream()))
+                           _p(state_slots), _p(cu_q), B, C, taps, _p(in_bias), _stream()))
 
 
 def gated_group_norm(y: torch.Tensor, x: torch.Tensor, skip: torch.Tensor, z: torch.Tensor, weight: torch.Tensor, eps: float,
@@ -2113,4 +2143,273 @@ def rows_rmsnorm(x: torch.Tensor, weight: Optional[torch.Tensor], eps: float, ou
     stride = int(x.stride(0)) if T > 1 else n
     _ok(lib().xi_rows_rmsnorm(_p(x), ctypes.c_longlong(stride), _code(x, "rows_rmsnorm"), _p(weight), ctypes.c_float(eps), _p(out),
                               _code(out, "rows_rmsnorm"), int(T), int(n), _stream()))
+    return out
+
+
+# ---- recurrences of one number a channel ---------------------------------------------------------------------------------
+CHANNEL_CHUNK = 32            # least tokens of a chunk of a long portion (0: every portion is walked in one piece)
+CHANNEL_CHUNKS = 64           # chunks a step's tokens are cut into at most, about: longer steps get longer chunks
+
+
+def channel_chunk(tokens: int) -> int:
+    """Tokens a chunk of `channel_scan` for a step of so many tokens (a multiple of the walk's eight)."""
+    return 0 if CHANNEL_CHUNK <= 0 else max(CHANNEL_CHUNK, -(-int(tokens) // CHANNEL_CHUNKS // 8) * 8)
+
+
+def channel_items(q_lens, chunk: int):
+    """The items a step's portions are walked in: rows (first token, last token, batch row, the portion's first item, its
+    items), a portion of two chunks and more in as many items, the others in one each."""
+    whole, long, chunks = scan_chunk_plan(q_lens, chunk)
+    cut = {b: (c0, n) for b, c0, n in long}
+    rows, at = [], 0
+    for b, n in enumerate(q_lens):
+        lead = len(rows)
+        if b in cut:
+            c0, count = cut[b]
+            for first, size in chunks[c0:c0 + count]:
+                rows.append((at + first, at + first + size, b, lead, count))
+        else:
+            rows.append((at, at + int(n), b, lead, 1))
+        at += int(n)
+    return rows
+
+
+def channel_scan(gate: torch.Tensor, gate_act: str, state: torch.Tensor, state_slots: torch.Tensor, cu_q: torch.Tensor,
+                 ready=None, mingru=None, gate_bias: Optional[torch.Tensor] = None, q_lens=None, plan_cache=None) -> torch.Tensor:
+    """S_t = a_t S_(t-1) + b_t channel by channel from the state each request's slot holds (float32 [slots, C], left there
+    afterwards); returns S_t * act(gate_t + gate_bias) [T, C] in the gate's type, act "silu", "gelu_tanh" or "none".
+    `ready` = (a, b) float32 [T, C], or `mingru` = (z, z_bias, u, u_bias): columns of one packed projection in the gate's
+    type and float32 [C] biases (or None), a = 1 - sigmoid(z), b = sigmoid(z) * (u + 1/2 where u >= 0, sigmoid(u) where
+    u < 0).  `q_lens` and `plan_cache` as for `linear_scan`: long portions are walked in chunks side by side."""
+    T, C = gate.shape
+    gs = _columns(gate, C, "channel_scan: gate")
+    acts = {"none": 0, "silu": 1, "gelu_tanh": 2}
+    if gate_act not in acts or (ready is None) == (mingru is None):
+        raise KernelError("channel_scan: a known activation, and ready-made terms or minGRU columns")
+    a = b = z = u = zb = ub = None
+    zs = 0
+    if ready is not None:
+        a, b = ready
+        for t in (a, b):
+            _want(t, torch.float32, "channel_scan: a and b")
+            if tuple(t.shape) != (T, C):
+                raise KernelError(f"channel_scan: terms {tuple(t.shape)} are not [{T}, {C}]")
+    else:
+        z, zb, u, ub = mingru
+        zs, us = _columns(z, C, "channel_scan: z"), _columns(u, C, "channel_scan: u")
+        if zs != us or z.shape[0] != T or u.shape[0] != T or z.dtype != gate.dtype or u.dtype != gate.dtype:
+            raise KernelError("channel_scan: z and u must be columns of the same rows as the gate")
+    _dev(a, b, zb, ub, gate_bias, state_slots, cu_q)
+    for t in (zb, ub, gate_bias):
+        if t is not None and (t.dtype != torch.float32 or t.shape != (C,)):
+            raise KernelError(f"channel_scan: biases must be float32 [{C}]")
+    _want(state, torch.float32, "channel_scan: state")
+    _want(state_slots, torch.int64, "channel_scan: state_slots")
+    _want(cu_q, torch.int32, "channel_scan: cu_q")
+    B = state_slots.shape[0]
+    if state.dim() != 2 or state.shape[1] != C or state.stride(1) != 1 or not state.is_cuda or cu_q.shape != (B + 1,):
+        raise KernelError(f"channel_scan: state [slots, {C}] and cu_q [B + 1] expected")
+    if q_lens is not None and (len(q_lens) != B or sum(int(n) for n in q_lens) != T):
+        raise KernelError("channel_scan: the portions' lengths do not add up to the step's tokens")
+    items, n, share, init = None, B, None, None
+    if q_lens is not None:
+        key = ("channel_scan_items", CHANNEL_CHUNK, CHANNEL_CHUNKS)
+        plan = plan_cache.get(key) if plan_cache is not None else None
+        if plan is None:
+            rows = channel_items(q_lens, channel_chunk(T))
+            plan = (torch.tensor(rows, dtype=torch.int32).to(gate.device) if len(rows) > B else None, len(rows))
+            if plan_cache is not None:
+                plan_cache[key] = plan
+        items, n = plan
+    if items is not None:
+        share = torch.empty((n, 2, C), dtype=torch.float32, device=gate.device)
+        init = torch.empty((n, C), dtype=torch.float32, device=gate.device)
+    out = torch.empty((T, C), dtype=gate.dtype, device=gate.device)
+    stride = int(state.stride(0)) if state.shape[0] > 1 else C
+    ll = ctypes.c_longlong
+    _ok(lib().xi_channel_scan(_p(a), _p(b), _p(z), _p(u), ll(zs), _p(zb), _p(ub), _p(gate), ll(gs), _p(gate_bias), acts[gate_act],
+                              _p(state), ll(stride), _p(state_slots), _p(cu_q), _p(items), int(n), int(items is not None), _p(share),
+                              _p(init), _p(out), _code(gate, "channel_scan"), C, _stream()))
+    return out
+
+
+RGLRU_MFMA = True         # False: bfloat16 gates go through the vector kernels too
+
+
+def rglru_terms(u: torch.Tensor, weight: torch.Tensor, r_bias: torch.Tensor, i_bias: torch.Tensor, rate: torch.Tensor):
+    """(a, b) float32 [T, C] of a real-gated linear recurrent unit: with r, i the block-diagonal products of u [T, C]
+    (weight [blocks, 2, C / blocks, C / blocks], [out, in], the r gate's matrix first, in u's type) plus their biases, log a =
+    rate * sigmoid(r), a = exp(log a), b = sqrt(1 - a^2) * sigmoid(i) * u.  Biases and rate float32 [C]."""
+    _dev(u, weight, r_bias, i_bias, rate)
+    if u.dim() != 2 or weight.dim() != 4 or weight.shape[1] != 2 or weight.shape[2] != weight.shape[3] or weight.dtype != u.dtype:
+        raise KernelError("rglru_terms: u [T, C] and weight [blocks, 2, n, n] of one type")
+    T, C = u.shape
+    blocks, per = int(weight.shape[0]), int(weight.shape[2])
+    if blocks * per != C:
+        raise KernelError(f"rglru_terms: {blocks} blocks of {per} for {C} channels")
+    for t in (r_bias, i_bias, rate):
+        _want(t, torch.float32, "rglru_terms: biases and rate")
+        if t.shape != (C,):
+            raise KernelError(f"rglru_terms: biases and rate must be [{C}]")
+    a = torch.empty((T, C), dtype=torch.float32, device=u.device)
+    b = torch.empty((T, C), dtype=torch.float32, device=u.device)
+    if u.dtype == torch.bfloat16 and per % 8 == 0 and RGLRU_MFMA:
+        _ok(lib().xi_rglru_gates(_p(u), _p(weight), _p(r_bias), _p(i_bias), _p(rate), _p(a), _p(b), T, C, per, _stream()))
+        return a, b
+    logits = torch.empty((T, blocks, 2 * per), dtype=torch.float32, device=u.device)
+    head_linear(u.view(T, blocks, per), weight.view(blocks, 2 * per, per), logits)
+    _ok(lib().xi_rglru_terms(_p(logits), _p(r_bias), _p(i_bias), _p(rate), _p(u), _code(u, "rglru_terms"), _p(a), _p(b), T, C, per,
+                             _stream()))
+    return a, b
+
+
+def row_norm_gate(o: torch.Tensor, weight: torch.Tensor, eps: float, gate: torch.Tensor, act: str = "sigmoid") -> torch.Tensor:
+    """o float32 [T, W]: each row divided by its root mean square (eps inside the root), times `weight` float32 [W], times
+    sigmoid(gate) or silu(gate) (gate [T, W], may be a column range of a packed projection).  In the gate's type."""
+    _dev(o, weight)
+    _want(o, torch.float32, "row_norm_gate: o")
+    _want(weight, torch.float32, "row_norm_gate: weight")
+    T, W = o.shape
+    gs = _columns(gate, W, "row_norm_gate: gate")
+    if gate.shape[0] != T or gate.device != o.device or weight.shape != (W,) or act not in ("sigmoid", "silu"):
+        raise KernelError(f"row_norm_gate: gate rows of the same tokens, weight [{W}], act sigmoid or silu")
+    out = torch.empty((T, W), dtype=gate.dtype, device=o.device)
+    _ok(lib().xi_row_norm_gate(_p(o), _p(weight), ctypes.c_float(eps), _p(gate), ctypes.c_longlong(gs), int(act == "sigmoid"), _p(out),
+                               _code(gate, "row_norm_gate"), T, W, _stream()))
+    return out
+
+
+# ---- what the stream is still to get, and what is read of it -----------------------------------------------------------------
+JOIN_PLAIN, JOIN_NORMED, JOIN_NORMS = 3, 2, 2         # terms without and with a norm, and norms of the new row, of one launch
+
+
+def stream_join(x: Optional[torch.Tensor], terms=(), norms=(), out_dtype: torch.dtype = torch.float32,
+                keep: bool = False, result: Optional[torch.Tensor] = None, rounded: bool = False, average=None,
+                rows: Optional[torch.Tensor] = None, shape=None):
+    """s = x + sum over `terms` (y, weight, eps, factor) of factor * y, a term with a weight (float32 [H]) as factor * (y /
+    sqrt(mean(y^2) + eps)) * weight; y rows [T, H] in either precision or a stack [P, T, H] of float32 partial sums.  With
+    `average` = (first [T, H], past [N, T, H], n, coef [n + 2]): u = coef[0] first + sum_(j < n) coef[1 + j] past[j] + coef[n +
+    1] s, else u = s.  Returns (s or None, s rounded to out_dtype or None, u or None, [u / sqrt(mean(u^2) + eps) * weight in
+    out_dtype for the (weight, eps) of `norms`]).  `keep`: s is wanted (in `result`, a float32 [T, H] that is no operand, if
+    given); `rounded`: its rounding is; u comes back where there is an average and no `rows`.  `rows` int32: only those
+    rows are made, and only the norms.  x None (with `shape` = (T, H)): zeros."""
+    terms, norms = list(terms), list(norms)
+    T, H = x.shape if x is not None else shape
+    dev = x.device if x is not None else terms[0][0].device
+    if x is not None:
+        _want(x, torch.float32, "stream_join: the stream")
+    if rows is not None:
+        _want(rows, torch.int32, "stream_join: rows")
+        if keep or rounded or not norms:
+            raise KernelError("stream_join: with rows only norms are made")
+    if len(norms) > JOIN_NORMS or sum(t[1] is None for t in terms) > JOIN_PLAIN or sum(t[1] is not None for t in terms) > JOIN_NORMED:
+        raise KernelError("stream_join: too many terms or norms for one launch")
+    _dev(x, rows, result, *(t[0] for t in terms), *(t[1] for t in terms), *(n[0] for n in norms))
+    stride = 0
+    ys, codes, parts = [], [], []
+    for y, w, _, _ in terms:
+        p = 1
+        if y.dim() == 3:
+            _want(y, torch.float32, "stream_join: partial sums")
+            p, stride = int(y.shape[0]), T * H
+        if tuple(y.shape[-2:]) != (T, H) or y.dim() not in (2, 3) or p < 1:
+            raise KernelError(f"stream_join: a term {tuple(y.shape)} does not fit the stream {(T, H)}")
+        ys.append(y)
+        codes.append(_code(y, "stream_join"))
+        parts.append(p)
+    for w in [t[1] for t in terms] + [n[0] for n in norms]:
+        if w is not None and (w.dtype != torch.float32 or w.shape != (H,)):
+            raise KernelError(f"stream_join: weights must be float32 [{H}]")
+    first = past = coef = None
+    n_past = 0
+    if average is not None:
+        first, past, n_past, coef = average
+        _dev(first, past, coef)
+        for t in (first, coef) + ((past,) if n_past else ()):
+            _want(t, torch.float32, "stream_join: the average's operands")
+        if tuple(first.shape) != (T, H) or coef.shape != (int(n_past) + 2,) or (
+                n_past and (past.dim() != 3 or tuple(past.shape[1:]) != (T, H) or past.shape[0] < n_past)):
+            raise KernelError(f"stream_join: the average's results must be [{T}, {H}] each, its weights [{n_past} + 2]")
+    n = T if rows is None else int(rows.shape[0])
+    if result is not None and (tuple(result.shape) != (T, H) or result.dtype != torch.float32):
+        raise KernelError("stream_join: the result's place must be float32 [T, H]")
+    if keep and result is None:
+        result = torch.empty((T, H), dtype=torch.float32, device=dev)
+    elif not keep:
+        result = None
+    low = torch.empty((T, H), dtype=out_dtype, device=dev) if rounded else None
+    u = torch.empty((T, H), dtype=torch.float32, device=dev) if average is not None and rows is None else None
+    outs = [torch.empty((n, H), dtype=out_dtype, device=dev) for _ in norms]
+    k = len(terms)
+    voids = lambda ts: (ctypes.c_void_p * max(1, len(ts)))(*[None if t is None else t.data_ptr() for t in ts])
+    floats = lambda fs: (ctypes.c_float * max(1, len(fs)))(*fs)
+    ints = lambda vs: (ctypes.c_int * max(1, len(vs)))(*vs)
+    _ok(lib().xi_stream_join(_p(x), k, voids(ys), ints(codes), ints(parts), ctypes.c_longlong(stride), voids([t[1] for t in terms]),
+                             floats([t[2] for t in terms]), floats([t[3] for t in terms]), _p(result), _p(low), _p(first),
+                             _p(past if n_past else None), ctypes.c_longlong(T * H), int(n_past), _p(coef), _p(u), len(norms),
+                             voids([w for w, _ in norms]), floats([e for _, e in norms]), voids(outs),
+                             _CODE[out_dtype], _p(rows), n, H, _stream()))
+    return result, low, u, outs
+
+
+def embed_norm(table: torch.Tensor, ids: torch.Tensor, scale: float, weight: torch.Tensor, eps: float) -> torch.Tensor:
+    """x = float32(table[ids[t]]) * scale, out[t] = x / sqrt(mean(x^2) + eps) * weight, float32 [T, H]."""
+    _dev(table, ids, weight)
+    _want(ids, torch.int32, "embed_norm: ids")
+    _want(weight, torch.float32, "embed_norm: weight")
+    if table.dim() != 2 or ids.dim() != 1 or weight.shape != (table.shape[1],):
+        raise KernelError("embed_norm: table [V, H], ids [T], weight [H]")
+    T, H = ids.shape[0], table.shape[1]
+    out = torch.empty((T, H), dtype=torch.float32, device=table.device)
+    _ok(lib().xi_embed_norm(_p(table), _code(table, "embed_norm"), _p(ids), ctypes.c_float(scale), _p(weight), ctypes.c_float(eps), _p(out),
+                            T, H, _stream()))
+    return out
+
+
+# ---- a layer's own input for the token ---------------------------------------------------------------------------------------
+SIDE_GATE_TOKENS = 64         # steps of up to this many tokens make the gate's product inside the kernel that applies it
+
+
+def _side_table(table: torch.Tensor, offset: int, dim: int, ids: torch.Tensor, what: str) -> None:
+    _want(ids, torch.int32, f"{what}: ids")
+    if table.dim() != 2 or offset < 0 or offset + dim > table.shape[1] or ids.dim() != 1:
+        raise KernelError(f"{what}: a table [V, W] whose rows hold columns {offset} .. {offset + dim}, ids [T]")
+
+
+def side_mul(z: torch.Tensor, table: torch.Tensor, offset: int, ids: torch.Tensor) -> torch.Tensor:
+    """gelu_tanh(z[t]) * table[ids[t], offset : offset + dim] in the table's type; z [T, dim] in either precision or a stack
+    [P, T, dim] of float32 partial sums."""
+    _dev(z, table, ids)
+    parts = 1
+    if z.dim() == 3:
+        _want(z, torch.float32, "side_mul: partial sums")
+        parts = int(z.shape[0])
+    T, dim = int(z.shape[-2]), int(z.shape[-1])
+    _side_table(table, int(offset), dim, ids, "side_mul")
+    if ids.shape[0] != T:
+        raise KernelError("side_mul: a row of the gate for every token")
+    out = torch.empty((T, dim), dtype=table.dtype, device=table.device)
+    _ok(lib().xi_side_mul(_p(z), _code(z, "side_mul"), parts, ctypes.c_longlong(T * dim), _p(table), ctypes.c_longlong(int(table.shape[1])),
+                          int(offset), _p(ids), _p(out), _code(table, "side_mul"), T, dim, _stream()))
+    return out
+
+
+def side_gate_takes(T: int, K: int, dtype: torch.dtype) -> bool:
+    return dtype == torch.bfloat16 and 0 < T <= SIDE_GATE_TOKENS and K % 8 == 0
+
+
+def side_gate(x: torch.Tensor, weight: torch.Tensor, table: torch.Tensor, offset: int, ids: torch.Tensor) -> torch.Tensor:
+    """`side_mul` of z = x @ weight^T in one launch, for few tokens in bfloat16 (x [T, K], weight [dim, K], K a multiple of 8)."""
+    _dev(x, weight, table, ids)
+    if x.dtype != torch.bfloat16 or weight.dtype != torch.bfloat16 or table.dtype != torch.bfloat16:
+        raise KernelError("side_gate: operands must be bfloat16")
+    if x.dim() != 2 or weight.dim() != 2 or x.shape[1] != weight.shape[1] or x.shape[1] % 8:
+        raise KernelError(f"side_gate: x {tuple(x.shape)} and weight {tuple(weight.shape)} do not match")
+    T, K, dim = int(x.shape[0]), int(x.shape[1]), int(weight.shape[0])
+    _side_table(table, int(offset), dim, ids, "side_gate")
+    if ids.shape[0] != T:
+        raise KernelError("side_gate: an id for every token")
+    out = torch.empty((T, dim), dtype=torch.bfloat16, device=x.device)
+    _ok(lib().xi_side_gate(_p(x), _p(weight), _p(table), ctypes.c_longlong(int(table.shape[1])), int(offset), _p(ids), _p(out), T, dim, K,
+                           _stream()))
     return out

@@ -25,6 +25,11 @@ is, so the plain form computes this with its own kernels (norm with a weight of 
 rounding); with the options of the paragraph above, or with `general=True`, a kernel that takes a head at a time does
 it in the order given (`kernels.head_rows`: rotation of either pairing, then the unit norm, then the cache write).
 
+The general form also takes biases on q, k and v, the q/k norm head by head (before the rotation) and keys seen by chunks:
+with `chunk` c a query at position p sees the keys p - p mod c .. p (chunks counted from the sequence's first token; of such
+a layer the cache keeps the last c tokens, as of a window).  Values as long as the keys go through the plain form's fused kernel for the
+heads, others a head at a time (`kernels.head_rows`), and then the attention kernels that know the score's options.
+
 A third group of options, each a parameter of the spec, goes through `_forward_rows` (no rotation, `qk_norm` "row" or
 none): `conv` n: q, k and v pass a causal convolution per channel over the last n tokens right after the
 projection (tensors `q_conv`, `k_conv`, `v_conv` [channels, n], no bias; the last n - 1 projected rows of a request are
@@ -65,6 +70,9 @@ class PagedAttention(Mixer):
         self.qk_norm = bool(spec.get("qk_norm", False))
         self.qk_norm_eps = float(spec.get("qk_norm_eps", 1e-6))
         self.window = int(spec.get("window") or 0)
+        self.chunk = int(spec.get("chunk") or 0)
+        if self.window < 0 or self.chunk < 0:
+            raise ValueError(f"a window of {self.window} and chunks of {self.chunk} keys")
         self.scale = float(spec.get("scale", self.d ** -0.5))
         self.dv = int(spec.get("value_dim") or self.d)
         self.row_norm = spec.get("qk_norm") == "row"
@@ -81,14 +89,15 @@ class PagedAttention(Mixer):
         self.slopes = None           # float32 [nq] on the device
         # the options that the fused q/k kernel and the attention kernels of the plain form do not know
         self.general = bool(self.dv != self.d or self.row_norm or self.softcap > 0 or self.slope_values is not None
-                            or self.value_mix_key is not None or spec.get("general", False))
+                            or self.value_mix_key is not None or self.chunk > 0 or spec.get("general", False))
         interleaved = spec.get("position") is not None and bool(spec["position"].get("interleaved", False))
-        # the general form's heads are made ready a head at a time where they are normed one by one or turned in pairs
-        # (2i, 2i + 1); else a row at a time
-        self.by_head = self.general and (self.unit_norm or interleaved)
+        self.head_norm = self.qk_norm and not self.row_norm and not self.unit_norm          # a weight [head_dim], before the rotation
+        # the general form's heads are made ready a head at a time where they are normed one by one, turned in pairs
+        # (2i, 2i + 1) or have biases; else a row at a time
+        self.by_head = self.general and (self.unit_norm or self.head_norm or interleaved or self.bias)
         if self.by_head and (self.row_norm or self.value_mix_key is not None):
-            raise NotImplementedError("attention whose heads are normed one by one or turned in pairs (2i, 2i + 1) takes no "
-                                      "norm over the whole projection and no blended values")
+            raise NotImplementedError("attention whose heads are normed one by one, turned in pairs (2i, 2i + 1) or have biases "
+                                      "takes no norm over the whole projection and no blended values")
         self.taps = int(spec.get("conv") or 0)
         self.value_unit = spec.get("value_norm") == "head_unit"
         if spec.get("value_norm") not in (None, "head_unit"):
@@ -100,16 +109,12 @@ class PagedAttention(Mixer):
         if self.rows_form:
             self.general = True
             if (self.by_head or spec.get("position") is not None or self.softcap > 0 or self.slope_values is not None
-                    or self.value_mix_key is not None or self.bias or (self.qk_norm and not self.row_norm)):
+                    or self.value_mix_key is not None or self.chunk > 0 or self.bias or (self.qk_norm and not self.row_norm)):
                 raise NotImplementedError("attention with a convolution, normed values, mixed heads or a gate a head takes the "
-                                          "q/k norm over the whole projection or none, and no rotation, cap, bias or blend")
+                                          "q/k norm over the whole projection or none, and no rotation, cap, bias, chunks or blend")
         self.conv_w = self.talk = None
         if self.general and not self.by_head and spec.get("position") is not None and self.qk_norm:
-            raise NotImplementedError("attention with a soft cap, a distance bias, blended values or another value size takes a "
-                                      "rotation of the pairs (i, i + rotary_dim / 2) and then no q/k norm")
-        if self.general and (self.qk_norm and not (self.row_norm or self.unit_norm) or self.bias):
-            raise NotImplementedError("attention with a soft cap, a distance bias, blended values or another value size "
-                                      "takes the q/k norm over the whole projection, the heads' unit norm or none, and no biases")
+            raise NotImplementedError("a rotation and a norm over the whole projection")
         if self.nq % self.nkv:
             raise ValueError(f"{self.nq} query heads are not a multiple of {self.nkv} kv heads")
         # A step of single tokens reads nothing on the host where the split-K decode kernel or the
@@ -197,7 +202,8 @@ class PagedAttention(Mixer):
     # ---- cache ---------------------------------------------------------------
     def cache_need(self) -> KVNeed:
         # the matrix-core kernels of the bfloat16 path read V in groups of eight keys
-        need = KVNeed.keys_values(self.nkv, self.d, self.window, v_grouped=self.dtype == torch.bfloat16,
+        seen = min([n for n in (self.window, self.chunk) if n > 0], default=0)      # a chunk's keys are within its last `chunk` tokens
+        need = KVNeed.keys_values(self.nkv, self.d, seen, v_grouped=self.dtype == torch.bfloat16,
                                   value_dim=self.dv)
         if self.talking:           # mixed heads score against a token's whole k row: one key head of all kv heads' dims
             need = KVNeed(need.window, (PoolNeed("k", (1, PAGE, self.nkv * self.d)), need.pools[1]))
@@ -267,21 +273,33 @@ class PagedAttention(Mixer):
                 if v_other is None:
                     raise RuntimeError(f"values {self.value_mix_key!r} are blended in before the layer that makes them has run")
         pos = self.position
+        if self.by_head and self.dv == self.d and not self.unit_norm:      # the plain form's heads under another score
+            q = kernels.qk_norm_rope_kv(
+                qkv, self.q_norm_w, self.k_norm_w, self.qk_norm_eps,
+                pos.cos if pos is not None else ctx.empty_f32, pos.sin if pos is not None else ctx.empty_f32,
+                pos.rotary_dim if pos is not None else 0, pos.interleaved if pos is not None else False,
+                ctx.positions, slots, cache.k, cache.v, self.nq, self.nkv, self.d, v_grouped=vt,
+                vector_min_tokens=128 if ctx.max_q_len > 1 else self.VECTOR_MIN_DECODE, bias=self.qkv_bias)
+            a = kernels.attention(q, cache.k, cache.v, ctx, cache.group, self.scale, self.window, v_grouped=vt,
+                                  softcap=self.softcap, slopes=self.slopes, chunk=self.chunk)
+            return self.o(a, out_dtype=self.dtype, allow_split=True, sink=sink)
         if self.by_head:
             q = kernels.head_rows(qkv, slots, cache.k, cache.v, self.nq, self.nkv, self.d, self.dv, v_grouped=vt,
                                   cos=pos.cos if pos is not None else None, sin=pos.sin if pos is not None else None,
                                   rotary_dim=pos.rotary_dim if pos is not None else 0,
                                   interleaved=pos.interleaved if pos is not None else False, positions=ctx.positions,
-                                  unit_norm=self.unit_norm, eps=self.qk_norm_eps)
+                                  unit_norm=self.unit_norm, eps=self.qk_norm_eps, bias=self.qkv_bias,
+                                  q_weight=self.q_norm_w if self.head_norm else None,
+                                  k_weight=self.k_norm_w if self.head_norm else None)
             a = kernels.attention(q, cache.k, cache.v, ctx, cache.group, self.scale, self.window, v_grouped=vt,
-                                  softcap=self.softcap, slopes=self.slopes)
+                                  softcap=self.softcap, slopes=self.slopes, chunk=self.chunk)
             return self.o(a, out_dtype=self.dtype, allow_split=True, sink=sink)
         q = kernels.qkv_rows(qkv, self.q_norm_w, self.k_norm_w, self.qk_norm_eps, slots, cache.k, cache.v,
                              self.nq, self.nkv, self.d, self.dv, v_grouped=vt, v_other=v_other, mix=self.mix,
                              cos=pos.cos if pos is not None else None, sin=pos.sin if pos is not None else None,
                              rotary_dim=pos.rotary_dim if pos is not None else 0, positions=ctx.positions)
         a = kernels.attention(q, cache.k, cache.v, ctx, cache.group, self.scale, self.window, v_grouped=vt,
-                              softcap=self.softcap, slopes=self.slopes)
+                              softcap=self.softcap, slopes=self.slopes, chunk=self.chunk)
         return self.o(a, out_dtype=self.dtype, allow_split=True, sink=sink)
 
     def _forward_rows(self, x, ctx: StepContext, cache: LayerCache):

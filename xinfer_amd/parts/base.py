@@ -26,7 +26,8 @@ runs on the tokens of one step.  A part never learns which model it is in.
   Head             forward(h) -> float32 logits [R, vocab]; load(..., shared=) takes the
                    embedding's table when the spec says `tied`
   StreamOp         forward(stream, first, ctx) -> stream: a change of the stream between two runs
-                   of layers (what a pass over a span of layers adds when it starts)
+                   of layers (what a pass over a span of layers adds when it starts, what a layer
+                   adds behind its branches, an average over the layers so far)
 
 New kinds register themselves with the decorators below; a `PartSpec.kind` then selects
 them.  Nothing else in the engine has to change.
@@ -149,6 +150,7 @@ class StepContext:
     no_slots: Optional[torch.Tensor] = None    # int64 [T] of -1: "store nothing"
     empty_f32: Optional[torch.Tensor] = None   # float32 [1, 0]: tables of "no rotation"
     scratch: Dict[Any, Any] = field(default_factory=dict)   # per-step data that kernels derive once
+    ids: Optional[torch.Tensor] = None         # int32 [T]   the step's token ids (set by the model)
 
 
 @dataclass
@@ -177,17 +179,46 @@ class Folded:
 
 
 @dataclass
+class Term:
+    """Something the stream is to get: scale * y, or with a `weight` (float32 [H]) scale * (y / sqrt(mean(y^2) + eps)) *
+    weight.  y: rows in either precision, or a stack [P, T, H] of float32 partial sums."""
+    y: torch.Tensor
+    weight: Optional[torch.Tensor] = None
+    eps: float = 0.0
+    scale: float = 1.0
+
+
+@dataclass
+class DepthAverage:
+    """What is to become of the stream once its terms are added: the sum s is the `place`-th result of the layers (kept in
+    `results` [N, T, H], after the `place` results before it), and the stream becomes weights[0] first + sum over the results
+    before of weights[1 + j] results[j] + weights[place + 1] s (`first`: the embedding's output)."""
+    first: torch.Tensor
+    results: torch.Tensor
+    place: int
+    weights: torch.Tensor
+
+
+@dataclass
 class Stream:
     """The residual stream between blocks: `resid` float32 [T, H], and a branch output
     `pending` that has not been added to it yet (the next norm adds it in the same
     kernel that norms), or `folded`: the branch output is already added and the next
-    norm (`folded.norm`) half done."""
+    norm (`folded.norm`) half done.  A stream with `terms` or an `average` is `open`: who reads it next
+    adds them (`parts.joining.join`, which can norm the new rows in the same pass); parts that know
+    nothing of it are given a joined one."""
     resid: torch.Tensor
     pending: Optional[torch.Tensor] = None
     folded: Optional[Folded] = None
     rows: Optional[torch.Tensor] = None       # `resid` rounded to the activation dtype, as it is now (nothing
                                               # pending): what a sublayer that reads the stream itself takes
     pending_scale: float = 1.0                # the stream is to get pending_scale * pending
+    terms: Tuple[Term, ...] = ()              # what it is to get besides
+    average: Optional[DepthAverage] = None    # and what is then to become of it
+
+    @property
+    def open(self) -> bool:
+        return bool(self.terms) or self.average is not None
 
 
 class Part:
@@ -225,6 +256,11 @@ class Mixer(Part):
 
     def forward(self, x: torch.Tensor, ctx: StepContext, cache: LayerCache) -> torch.Tensor:
         raise NotImplementedError
+
+    def forward_terms(self, x: torch.Tensor, ctx: StepContext, cache: LayerCache) -> Tuple["Term", ...]:
+        """The result as terms whose sum it is, for blocks that add them in a pass of their own; a mixer that ends in
+        a sum of (normed) branches can hand those on."""
+        return (Term(self.forward(x, ctx, cache)),)
 
 
 class FeedForward(Part):
@@ -265,10 +301,12 @@ class TokenEmbedding(Part):
 
 
 class StreamOp(Part):
-    """Something that changes the residual stream between two runs of layers (`ScheduleEntry.before`):
+    """Something that changes the residual stream between two runs of layers (`ScheduleEntry.before` and `after`):
     forward(stream, first, ctx) -> stream, with `first` the embedding's output as it was before the first layer
     (float32 [T, H]; None unless the kind says `needs_first`)."""
     needs_first = False
+    writes_stream = True       # `forward` may change the stream's tensor in place
+    takes_open = False         # `forward` takes a stream that is `open`
 
     def forward(self, stream: "Stream", first: Optional[torch.Tensor], ctx: StepContext) -> "Stream":
         raise NotImplementedError
@@ -288,6 +326,8 @@ class Block:
     """Arrangement of a layer's parts around the residual stream."""
 
     graph_safe = False
+    writes_stream = True       # `forward` may change the stream's tensor in place
+    takes_open = False         # `forward` takes a stream that is `open` (see `Stream`)
 
     def __init__(self, layer: LayerSpec, dtype: torch.dtype):
         self.layer = layer

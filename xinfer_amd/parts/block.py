@@ -11,6 +11,10 @@ without a feed-forward ends after the first of the two.
 "branchnorm": x <- x + norm1(mixer(x)); x <- x + norm2(ff(x)): the sublayers read the stream
 itself and their OUTPUT is normed; a layer may have no feed-forward.  The norm, the add and
 the rounding of the new stream for the next sublayer are one kernel (`Norm.forward_branch`).
+
+"parallel": x <- x + (mixer(norm1(x)) + ff(norm2(x))), both of the same x, each with a norm of its own; a layer may have
+no feed-forward.  One pass makes x (what the layers before left to be added) and both normed rows; the two branches are
+left to be added by whoever reads the stream next (`Stream.terms`).
 """
 from __future__ import annotations
 
@@ -21,8 +25,9 @@ import torch
 from .. import kernels
 from ..config.spec import LayerSpec
 from ..weights.store import TensorDecl, WeightStore
-from .base import (Block, Folded, KVNeed, LayerCache, NormSink, StateNeed, StepContext, Stream,
+from .base import (Block, Folded, KVNeed, LayerCache, NormSink, StateNeed, StepContext, Stream, Term,
                    feed_forward_class, mixer_class, norm_class, register_block)
+from .joining import join, joins
 
 @register_block("prenorm")
 class PreNormBlock(Block):
@@ -187,3 +192,58 @@ class BranchNormBlock(Block):
             m = self.ffn.forward(x if rows_dtype is not None else resid, ctx)
             x = self.norms[1].forward_branch(resid, m, rows_dtype)
         return Stream(resid, None, None, rows=x)
+
+
+@register_block("parallel")
+class ParallelBlock(Block):
+    """`layer.norms` names the norm before the mixer first, then the one before the feed-forward."""
+    writes_stream = False
+    takes_open = True
+
+    def __init__(self, layer: LayerSpec, dtype: torch.dtype):
+        super().__init__(layer, dtype)
+        self.mixer = mixer_class(layer.mixer.kind)(layer.mixer, dtype)
+        self.ffn = (feed_forward_class(layer.feed_forward.kind)(layer.feed_forward, dtype)
+                    if layer.feed_forward is not None else None)
+        items = layer.norm_items(2 if self.ffn is not None else 1)
+        self._names = [n for n, _ in items]
+        self.norms = [norm_class(n.kind)(n, dtype) for _, n in items]
+
+    @classmethod
+    def declare(cls, layer: LayerSpec) -> List[TensorDecl]:
+        p = layer.prefix
+        out = mixer_class(layer.mixer.kind).declare(layer.mixer, f"{p}.{layer.mixer_name}")
+        if layer.feed_forward is not None:
+            out += feed_forward_class(layer.feed_forward.kind).declare(layer.feed_forward, f"{p}.{layer.feed_forward_name}")
+        for name, n in layer.norm_items(2 if layer.feed_forward is not None else 1):
+            out += norm_class(n.kind).declare(n, f"{p}.{name}")
+        return out
+
+    def load(self, store: WeightStore, device) -> None:
+        p = self.layer.prefix
+        self.mixer.load(store, f"{p}.{self.layer.mixer_name}", device)
+        if self.ffn is not None:
+            self.ffn.load(store, f"{p}.{self.layer.feed_forward_name}", device)
+        for name, norm in zip(self._names, self.norms):
+            norm.load(store, f"{p}.{name}", device)
+
+    @property
+    def graph_safe(self) -> bool:
+        return all(p.graph_safe for p in (self.mixer, *self.norms, *(() if self.ffn is None else (self.ffn,))))
+
+    def cache_need(self) -> Optional[KVNeed]:
+        return self.mixer.cache_need()
+
+    def state_need(self) -> Optional[StateNeed]:
+        return self.mixer.state_need()
+
+    def forward(self, stream: Stream, ctx: StepContext, cache: LayerCache) -> Stream:
+        if joins(*self.norms):
+            stream, _, rows = join(stream, self.dtype, self.norms)
+        else:
+            stream = join(stream, self.dtype)[0]
+            rows = [n.forward(stream.resid, None, self.dtype) for n in self.norms]
+        terms = tuple(self.mixer.forward_terms(rows[0], ctx, cache))
+        if self.ffn is not None:
+            terms += (Term(self.ffn.forward(rows[1], ctx)),)
+        return Stream(stream.resid, terms=terms)

@@ -7,6 +7,8 @@ With `pairs` (name, buckets, mul_prev, mul_cur) a row of a second table [buckets
 token and the one before it: row (prev * mul_prev + token * mul_cur) mod buckets, and the last row for a sequence's
 first token.  The token before is state of the request: the embedding keeps one int32 a live request
 (`state_need`), written after every step, so a prompt may be cut anywhere.
+With `norm` (eps, name, weight_offset) the result is divided by its root mean square over dim and multiplied by
+weight_offset + the tensor `name` (float32; the start of the stream is then the normed row).
 "lm_head": logits = h @ W^T in float32; W is the embedding table when the spec says `tied`
 (qwen3.rs:267-287,367-373); `scale` s, if the spec gives one, multiplies them; `softcap` c, if the spec
 gives one, then makes them c * tanh(logits / c).
@@ -45,12 +47,20 @@ class Embedding(TokenEmbedding):
         if self.pairs is not None and self.sinusoid_base > 0:
             raise NotImplementedError("an embedding with sinusoidal positions and a table of pairs")
         self.pair_table: Optional[torch.Tensor] = None
+        norm = spec.get("norm")
+        self.norm = None if not norm else dict(name=str(norm["name"]), eps=float(norm["eps"]), offset=float(norm.get("weight_offset") or 0.0))
+        self.norm_w: Optional[torch.Tensor] = None
+        if self.norm is not None and (self.pairs is not None or self.sinusoid_base > 0):
+            raise NotImplementedError("a normed embedding with a table of pairs or sinusoidal positions")
 
     @classmethod
     def declare(cls, spec: PartSpec, prefix: str = "") -> List[TensorDecl]:
         out = [TensorDecl(spec["name"], (int(spec["vocab_size"]), int(spec["dim"])))]
         if spec.get("pairs"):
             out.append(TensorDecl(spec["pairs"]["name"], (int(spec["pairs"]["buckets"]) + 1, int(spec["dim"]))))
+        if spec.get("norm"):
+            offset = float(spec["norm"].get("weight_offset") or 0.0)
+            out.append(TensorDecl(spec["norm"]["name"], (int(spec["dim"]),), f"normal({1.0 - offset},0.1)" if offset else "norm"))
         return out
 
     def state_need(self) -> Optional[StateNeed]:
@@ -63,6 +73,8 @@ class Embedding(TokenEmbedding):
         self.table = t.contiguous()
         if self.pairs is not None:
             self.pair_table = store.get(self.pairs["name"], None, device).to(self.table.dtype).contiguous()
+        if self.norm is not None:
+            self.norm_w = (store.get(self.norm["name"], torch.float32, device) + self.norm["offset"]).contiguous()
         if self.sinusoid_base > 0:
             i = torch.arange((self.dim + 1) // 2, dtype=torch.float32)
             self.freq = (torch.tensor(self.sinusoid_base, dtype=torch.float32) ** (-2.0 * i / self.dim)).to(device).contiguous()
@@ -76,6 +88,8 @@ class Embedding(TokenEmbedding):
                                      cache.state, self.scale, p["buckets"], p["mul_prev"], p["mul_cur"])
             kernels.keep_last_token(ids, ctx.cu_q, ctx.state_slots, cache.state)
             return out
+        if self.norm is not None:
+            return kernels.embed_norm(self.table, ids, self.scale, self.norm_w, self.norm["eps"])
         if self.freq is None:
             return kernels.embed(self.table, ids, scale=self.scale)
         if ctx is None:

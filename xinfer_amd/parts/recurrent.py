@@ -1,11 +1,11 @@
-"""Linear attention with a decaying state, as mixers: "gated_linear_attention" and "retention".
+"""Linear attention with a decaying state, as mixers: "gated_linear_attention", "retention" and "lightning_attention".
 
-Both keep, per request and head, a float32 matrix S [key_dim, value_dim] in the request's state slot
+All keep, per request and head, a float32 matrix S [key_dim, value_dim] in the request's state slot
 (no pages: the cache of such a layer does not grow with the context) and do, token by token,
 
     S <- diag(a_t) S + k_t v_t^T        o_t = S^T q_t
 
-then norm each head's o by its root mean square over value_dim (eps inside the root), multiply by
+then (the first two) norm each head's o by its root mean square over value_dim (eps inside the root), multiply by
 silu(g) with g a projection of the input of its own, and project the concatenated heads (`o`).  A state
 slot holds zeros when a request runs its first token (the runner clears it), and a step leaves the state
 after its last token there, so a prompt may be cut anywhere.
@@ -16,6 +16,9 @@ after its last token there, so a prompt may be cut anywhere.
                            by the heads.
   retention                a_t = decay[h], one constant a head; k is multiplied by `k_scale`
                            (key_dim^-1/2 unless given); the heads' norm has no weight.
+  lightning_attention      a_t = decay[h]; q, k and v pass silu and are not scaled; the concatenated heads are normed
+                           together (one root mean square over heads * value_dim, a weight of that length) and
+                           multiplied by sigmoid(g).
 
 Decays, their logarithms and exponentials, the state, o and its norm are float32 in both precisions; the
 projections and the gate's activation run in the activation dtype.  q, k, v and g are one packed
@@ -162,3 +165,33 @@ class Retention(_DecayingState):
         o = kernels.linear_scan(q, k, v, self._state(cache), ctx.state_slots, ctx.cu_q, self.heads, self.dk, self.dv,
                                 head_decay=self.decay, k_scale=self.k_scale, **self._cutting(ctx))
         return self.o(kernels.head_norm_gate(o, None, self.eps, g, self.dtype), out_dtype=self.dtype)
+
+
+@register_mixer("lightning_attention")
+class LightningAttention(_DecayingState):
+    NAMES = {**_DecayingState.NAMES, "norm": "norm"}
+
+    def __init__(self, spec: PartSpec, dtype: torch.dtype):
+        super().__init__(spec, dtype)
+        self.decay_values = tuple(float(d) for d in spec["decay"])
+        if len(self.decay_values) != self.heads:
+            raise ValueError(f"{len(self.decay_values)} decays for {self.heads} heads")
+        self.decay = self.norm_w = None
+
+    @classmethod
+    def declare(cls, spec: PartSpec, prefix: str) -> List[TensorDecl]:
+        n = cls._names(spec, prefix)
+        return cls._declare_common(spec, prefix) + [TensorDecl(n["norm"], (int(spec["num_heads"]) * int(spec["value_dim"]),), "norm")]
+
+    def load(self, store: WeightStore, prefix: str, device) -> None:
+        n = self._load_common(store, prefix, device)
+        self.decay = torch.tensor(self.decay_values, dtype=torch.float32, device=device)
+        self.norm_w = store.get(n["norm"], torch.float32, device).contiguous()
+
+    def forward(self, x: torch.Tensor, ctx: StepContext, cache: LayerCache) -> torch.Tensor:
+        p = self.proj(x, out_dtype=self.dtype)
+        q, k, v, g = self._split(p)
+        o = kernels.linear_scan(q, k, v, self._state(cache), ctx.state_slots, ctx.cu_q, self.heads, self.dk, self.dv,
+                                head_decay=self.decay, silu=True, **self._cutting(ctx))
+        o = kernels.row_norm_gate(o.view(o.shape[0], self.heads * self.dv), self.norm_w, self.eps, g, "sigmoid")
+        return self.o(o, out_dtype=self.dtype, allow_split=True)

@@ -35,20 +35,24 @@ class RotaryEmbedding(PositionEncoding):
         self.interleaved = bool(spec.get("interleaved", False))
         if self.rotary_dim % 2 or not (0 < self.rotary_dim <= self.head_dim):
             raise ValueError(f"rotary_dim {self.rotary_dim} must be even and within head_dim {self.head_dim}")
+        self.precise = bool(spec.get("precise", False))      # angles, cos and sin in float64, rounded once
         self.cos = self.sin = None
 
     def load(self, store, prefix, device) -> None:
         scaling = self.spec.get("scaling")
         key = (self.rotary_dim, self.theta, self.max_positions, str(torch.device(device)),
-               tuple(sorted(scaling.items())) if scaling else None)
+               tuple(sorted(scaling.items())) if scaling else None, self.precise)
         if key not in _TABLES:
-            inv_freq, mscale = scaled_inv_freq(self.theta, self.rotary_dim, scaling)
-            pos = torch.arange(self.max_positions, dtype=torch.float32)
-            ang = pos[:, None] * torch.from_numpy(inv_freq)[None, :]          # float32 product
+            if self.precise:
+                inv_freq, mscale = precise_inv_freq(self.theta, self.rotary_dim, scaling)
+            else:
+                inv_freq, mscale = scaled_inv_freq(self.theta, self.rotary_dim, scaling)
+            pos = torch.arange(self.max_positions, dtype=torch.float64 if self.precise else torch.float32)
+            ang = pos[:, None] * torch.from_numpy(inv_freq)[None, :]          # a float32 product, unless `precise`
             cos, sin = ang.cos(), ang.sin()
             if mscale != 1.0:
                 cos, sin = cos * mscale, sin * mscale
-            _TABLES[key] = (cos.contiguous().to(device), sin.contiguous().to(device))
+            _TABLES[key] = (cos.float().contiguous().to(device), sin.float().contiguous().to(device))
         self.cos, self.sin = _TABLES[key]
 
 
@@ -116,17 +120,28 @@ def scaled_inv_freq(theta: float, rot: int, scaling) -> "tuple[np.ndarray, float
         # lo = max(floor(dim(fast)), 0), hi = min(ceil(dim(slow)), rot - 1) and r_i = clamp((i - lo) / max(hi - lo, 0.001),
         # 0, 1), frequency i is f_i / factor * r_i + f_i (1 - r_i), and cos and sin grow by 0.1 ln(factor) + 1.  Made in
         # float64 and rounded once.
-        factor = float(scaling["factor"])
-        f = np.power(np.float64(theta), -np.arange(0, rot, 2, dtype=np.float64) / rot)
-
-        def dim_of(turns: float) -> float:
-            return rot * math.log(orig / (2.0 * math.pi * float(turns))) / (2.0 * math.log(theta))
-
-        lo = max(math.floor(dim_of(scaling["fast"])), 0)
-        hi = min(math.ceil(dim_of(scaling["slow"])), rot - 1)
-        ramp = np.clip((np.arange(rot // 2, dtype=np.float64) - lo) / max(hi - lo, 0.001), 0.0, 1.0)
-        return (f / factor * ramp + f * (1.0 - ramp)).astype(f32), 0.1 * math.log(factor) + 1.0
+        freq, grow = precise_inv_freq(theta, rot, scaling)
+        return freq.astype(f32), grow
     raise ValueError(f"Unknown rope_type: {kind}")
+
+
+def precise_inv_freq(theta: float, rot: int, scaling) -> "tuple[np.ndarray, float]":
+    """(frequencies float64 [rot / 2], factor on cos and sin): theta^(-2i / rot), or blended along a ramp (kind "ramp", see
+    `scaled_inv_freq`)."""
+    f = np.power(np.float64(theta), -np.arange(0, rot, 2, dtype=np.float64) / rot)
+    if not scaling or scaling["kind"] == "default":
+        return f, 1.0
+    if scaling["kind"] != "ramp":
+        raise ValueError(f"no float64 tables for rope_type {scaling['kind']}")
+    factor, orig = float(scaling["factor"]), float(scaling["original"])
+
+    def dim_of(turns: float) -> float:
+        return rot * math.log(orig / (2.0 * math.pi * float(turns))) / (2.0 * math.log(theta))
+
+    lo = max(math.floor(dim_of(scaling["fast"])), 0)
+    hi = min(math.ceil(dim_of(scaling["slow"])), rot - 1)
+    ramp = np.clip((np.arange(rot // 2, dtype=np.float64) - lo) / max(hi - lo, 0.001), 0.0, 1.0)
+    return f / factor * ramp + f * (1.0 - ramp), 0.1 * math.log(factor) + 1.0
 
 
 # layers with the same rotary parameters share one pair of tables per device

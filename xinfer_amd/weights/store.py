@@ -97,6 +97,14 @@ class WeightStore:
         want = dtype if dtype is not None else _storage_dtype(t.dtype)
         return t.to(device=device, dtype=want)
 
+    def shared(self, name: str, dtype: Optional[torch.dtype] = None, device="cpu") -> torch.Tensor:
+        """`get`, contiguous, and the same tensor for every part that asks for it: a table that several layers read."""
+        kept = self.__dict__.setdefault("_kept", {})
+        key = (name, dtype, str(torch.device(device)))
+        if key not in kept:
+            kept[key] = self.get(name, dtype, device).contiguous()
+        return kept[key]
+
     def check(self, decls: Iterable[TensorDecl]) -> List[str]:
         """Raises one `WeightError` if a declared tensor is missing or has another shape.
         Returns the names of the tensors that no declaration asks for."""
