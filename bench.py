@@ -90,6 +90,7 @@ DESIGN_SIZES = {
     "4k-moe": dict(width=4096, heads=32, kv_heads=8, dim=128, vdim=128, ff=12288, window=2048, experts=8, top=2),
     "2k-v": dict(width=2048, heads=16, kv_heads=4, dim=64, vdim=128, ff=8192, window=512, experts=16, top=2),
     "1k-moe": dict(width=1024, heads=16, kv_heads=8, dim=128, vdim=128, ff=3072, window=1024, experts=8, top=2),
+    "2k-d": dict(width=2048, heads=16, kv_heads=4, dim=64, vdim=128, ff=8192, window=512, experts=0, top=0),
     # two kv heads: the heads' mix scores a query against both kv heads' dims at once (256 of them)
     "1k-g2": dict(width=1024, heads=16, kv_heads=2, dim=128, vdim=128, ff=3072, window=1024, experts=0, top=0),
     "4k-g2": dict(width=4096, heads=32, kv_heads=2, dim=128, vdim=128, ff=12288, window=2048, experts=0, top=0),
@@ -106,8 +107,14 @@ VUZAZEN_SIZES = ("1k-g2", "4k-g2", "4k-g2-moe")
 # heads (a quarter as many as the query heads, keys as wide as the attention's and values twice that), the taps
 VUZAZEN_LATENT = dict(kv_rank=192, rot_dim=64)
 VUZAZEN_TAPS = 4
-DESIGN_CHOICES = {"mufenex": (tuple(k for k in DESIGN_SIZES if "g2" not in k), "qwen3"), "lilalorn": (LILALORN_SIZES, "mufenex"),
-                  "debusun": (DEBUSUN_SIZES, "mufenex"), "vuzazen": (VUZAZEN_SIZES, "debusun")}
+TISOSUN_SIZES = ("1k", "4k", "2k-d")
+# Tisosun's own sizes at every width: recurrences as wide as the model (gates in as many blocks as there are query heads, 4
+# taps), the linear attention's heads as Lilalorn's, half of a head turned, a token input of 256 columns a layer
+TISOSUN_SIDE = 256
+TISOSUN_TAPS = 4
+DESIGN_CHOICES = {"mufenex": (tuple(k for k in DESIGN_SIZES if "g2" not in k and k != "2k-d"), "qwen3"), "lilalorn": (LILALORN_SIZES, "mufenex"),
+                  "debusun": (DEBUSUN_SIZES, "mufenex"), "vuzazen": (VUZAZEN_SIZES, "debusun"),
+                  "tisosun": (TISOSUN_SIZES, "mufenex")}
 DESIGN_VOCAB = 32000
 MODELS = {"0.6b": QWEN3_0_6B, "8b": QWEN3_8B, "14b": QWEN3_14B, "32b": QWEN3_32B}
 CONTEXT = 4096
@@ -245,7 +252,7 @@ def product(spec: str, dev="cuda:0") -> int:
 
 def design_compare(spec: str, layers, steps: int, warmup: int, batch: int, context: int, prefill_tokens: int,
                    family: str = "both", only: str = "all") -> int:
-    """Mufenex beside Qwen3, Lilalorn or Debusun beside Mufenex, or Vuzazen beside Debusun, at equal sizes: ms of the
+    """Mufenex beside Qwen3, Lilalorn, Debusun or Tisosun beside Mufenex, or Vuzazen beside Debusun, at equal sizes: ms of the
     prefill of one prompt and of a decode step."""
     import torch
     from xinfer_amd.engine import ModelRunner, StepEntry, build_model
@@ -281,6 +288,20 @@ def design_compare(spec: str, layers, steps: int, warmup: int, batch: int, conte
                      vocab_size=DESIGN_VOCAB, sliding_window=z["window"], max_position_embeddings=2 * context)
         if name == "mufenex":
             return {"mufenex": mufenex, "qwen3": qwen3}
+        if name == "tisosun":
+            # attention within chunks beside linear attention, a real-gated recurrence, the same again, a minGRU, in turn
+            sh = max(1, z["heads"] // 4)
+            par = {"left": dict(heads=z["heads"], kv_heads=z["kv_heads"], dim=z["dim"], vdim=z["vdim"], scale=z["dim"] ** -0.5,
+                                softcap=50.0, mask={"size": z["window"]},
+                                rot=dict(dims=z["dim"] // 2, base=500000.0,
+                                         scaling=dict(factor=8.0, original=8192, fast=32.0, slow=1.0))),
+                   "right": dict(heads=sh, dim=z["dim"], vdim=2 * z["dim"], decay=[0.95 + 0.049 * h / max(1, sh - 1) for h in range(sh)])}
+            kinds = [("parallel", par), ("rglru", dict(width=z["width"], blocks=z["heads"], conv=TISOSUN_TAPS)), ("parallel", par),
+                     ("mingru", dict(width=z["width"]))]
+            tisosun = {"architecture": "Tisosun", "vocab": DESIGN_VOCAB, "width": z["width"], "norm": {"eps": 1e-6},
+                       "token_side": {"dim": TISOSUN_SIDE}, "max_positions": 2 * context,
+                       "layers": [{"type": kinds[i % 4][0], "mixer": kinds[i % 4][1], "mlp": mlp} for i in range(layers)]}
+            return {"tisosun": tisosun, "mufenex": mufenex}
         if name in ("debusun", "vuzazen"):
             # layers of a latent, windowed attention, a state space and windowed attention again, in turn; all of them
             # are one span that runs once, so that the start of a pass is in the step
@@ -458,10 +479,10 @@ def main() -> int:
                     help="serving workloads: read every step's tokens on the host before the next step is planned")
     ap.add_argument("--product", default=None, metavar="M,N,K[,slices[,shape]]",
                     help="time one bfloat16 product alone in the many-row tiled kernel and in the vendor library")
-    ap.add_argument("--design", default=None, metavar="mufenex[:SIZE]|lilalorn[:SIZE]|debusun[:SIZE]|vuzazen[:SIZE]",
-                    help="time another model family beside its closest one (Mufenex beside Qwen3, Lilalorn or Debusun beside Mufenex) at equal sizes (a line of its own; --layers, --steps, "
+    ap.add_argument("--design", default=None, metavar="mufenex[:SIZE]|lilalorn[:SIZE]|debusun[:SIZE]|tisosun[:SIZE]|vuzazen[:SIZE]",
+                    help="time another model family beside its closest one (Mufenex beside Qwen3, Lilalorn, Debusun or Tisosun beside Mufenex, Vuzazen beside Debusun) at equal sizes (a line of its own; --layers, --steps, "
                          "--warmup, --batch, --context, --prefill-tokens and --only apply)")
-    ap.add_argument("--family", choices=["both", "debusun", "lilalorn", "mufenex", "qwen3", "vuzazen"], default="both",
+    ap.add_argument("--family", choices=["both", "debusun", "lilalorn", "mufenex", "qwen3", "tisosun", "vuzazen"], default="both",
                     help="--design: time one of the two families only (for profiling)")
     ap.add_argument("--peaks", action="store_true",
                     help="also measure what this card reaches on a read-only stream of 4 GiB and on one square "

@@ -273,7 +273,7 @@ class PagedAttention(Mixer):
                 if v_other is None:
                     raise RuntimeError(f"values {self.value_mix_key!r} are blended in before the layer that makes them has run")
         pos = self.position
-        if self.by_head and self.dv == self.d and not self.unit_norm:      # the plain form's heads under another score
+        if self.by_head and self.dv == self.d <= 256 and not self.unit_norm:      # the plain form's heads under another score
             q = kernels.qk_norm_rope_kv(
                 qkv, self.q_norm_w, self.k_norm_w, self.qk_norm_eps,
                 pos.cos if pos is not None else ctx.empty_f32, pos.sin if pos is not None else ctx.empty_f32,
