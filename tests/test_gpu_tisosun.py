@@ -279,19 +279,21 @@ def test_convolution_without_an_activation_behind_a_bias(C, taps, dtype):
 
 # ---- linear attention behind silu, heads normed together -----------------------------------------------------------------
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("chunk", [0, 16])
-@pytest.mark.parametrize("H,dk,dv", [(3, 12, 20), (1, 20, 20), (5, 6, 10), (2, 64, 96), (4, 16, 1000)])
+@pytest.mark.parametrize("chunk", [0, 16, 64])
+@pytest.mark.parametrize("H,dk,dv", [(3, 12, 20), (1, 20, 20), (5, 6, 10), (2, 64, 96), (3, 40, 136), (2, 136, 24), (1, 256, 264), (4, 16, 1000)])
 def test_lightning_attention_in_portions(H, dk, dv, chunk, dtype, monkeypatch):
+    """Token by token, in chunks of the walk, and (bfloat16, sizes in eights) in chunks on the matrix cores, whose last one may
+    be a single token; short portions beside long ones; decays from a half to one."""
     from xinfer_amd import kernels
     monkeypatch.setattr(kernels, "SCAN_CHUNK", chunk)
     dt, eps = TD[dtype], 1e-5
-    lens, cuts, slots = [70, 1, 45], [[2, 64, 1, 3], [1], [40, 1, 1, 3]], [3, 0, 2]
+    lens, cuts, slots = [170, 1, 45, 64], [[2, 164, 1, 3], [1], [40, 1, 1, 3], [31, 33]], [3, 0, 2, 4]
     g = torch.Generator().manual_seed(H * dk)
     a, b = H * dk, H * dv
     packed = [(torch.randn(n, 2 * a + 2 * b, generator=g)).to(dt) for n in lens]
-    decay = torch.linspace(0.6, 0.9995, H)
+    decay = torch.linspace(0.5, 1.0, H) if H > 1 else torch.tensor([0.97])
     w = 1 + 0.2 * torch.randn(b, generator=g)
-    state = torch.full((5, H, dk, dv), 7.0, device=DEV)
+    state = torch.full((6, H, dk, dv), 7.0, device=DEV)
     for s in slots:
         state[s] = 0
     got = [[] for _ in lens]
@@ -302,16 +304,46 @@ def test_lightning_attention_in_portions(H, dk, dv, chunk, dtype, monkeypatch):
         out = kernels.row_norm_gate(o.view(-1, b), w.to(DEV), eps, p[:, 2 * a + b:], "sigmoid")
         for i, (r, _, _) in enumerate(rows):
             got[r].append(out[_cu(rows)[i]:_cu(rows)[i + 1]].cpu())
-    assert float(state[1].min()) == 7.0 and float(state[4].max()) == 7.0
+    assert float(state[1].min()) == 7.0 and float(state[5].max()) == 7.0
+    rounded = dtype == "bfloat16" and chunk > 0            # q, k and v behind silu are rounded once on the matrix cores
     for r, n in enumerate(lens):
         p = packed[r].double()
         q, k, v = (plain.silu(t) for t in (p[:, :a].view(n, H, dk), p[:, a:2 * a].view(n, H, dk), p[:, 2 * a:2 * a + b].view(n, H, dv)))
         o, S = plain.decayed_state(q, k, v, [float(x) for x in decay])
         want = plain.rms_norm(o.reshape(n, b), eps, w.double()) * torch.sigmoid(p[:, 2 * a + b:])
         err = (torch.cat(got[r]).double() - want).abs().max(dim=1).values
-        bad = (err > (2e-5 if dtype == "float32" else 8e-3) * want.abs().max()).nonzero()
-        assert bad.numel() == 0, f"request {r}: first wrong token {int(bad[0])}"
-        assert (state[slots[r]].cpu().double() - S).abs().max() < 2e-5 * max(1.0, float(S.abs().max()))
+        bad = (err > (2e-5 if dtype == "float32" else 1.2e-2) * want.abs().max()).nonzero()
+        assert bad.numel() == 0, f"request {r}: first wrong token {int(bad[0])}: {float(err[int(bad[0])]):.2e} of {float(want.abs().max()):.2e}"
+        assert (state[slots[r]].cpu().double() - S).abs().max() < (4e-3 if rounded else 2e-5) * max(1.0, float(S.abs().max()))
+
+
+@pytest.mark.parametrize("H,dk,dv,silu", [(2, 64, 40, False), (3, 32, 128, True), (1, 128, 64, False)])
+def test_decayed_states_on_the_matrix_cores_keep_float32(H, dk, dv, silu, monkeypatch):
+    """Inputs that bfloat16 holds exactly: the chunks' results and states then agree with the plain walk far below
+    bfloat16's rounding, whatever decays multiply in between, and a key planted hundreds of tokens back is read."""
+    from xinfer_amd import kernels
+    T, a = 700, H * dk
+    g = torch.Generator().manual_seed(dk)
+    p = torch.randn(T, 2 * a + H * dv, generator=g) * 0.5
+    p[3, a:2 * a] = 6.0                                    # token 3's key and value stand out
+    p[3, 2 * a:] = 8.0
+    p = p.bfloat16()
+    decay = torch.tensor([0.9973, 0.62, 0.99991][:H])
+    act = (lambda t: plain.silu(t).bfloat16().double()) if silu else (lambda t: t)
+    q, k, v = (act(t) for t in (p[:, :a].double().view(T, H, dk), p[:, a:2 * a].double().view(T, H, dk), p[:, 2 * a:].double().view(T, H, dv)))
+    want, S = plain.decayed_state(q, 0.25 * k, v, [float(d) for d in decay])
+    state = torch.zeros(2, H, dk, dv, device=DEV)
+    outs, at = [], 0
+    for n in (40, 1, 459, 200):
+        rows = p[at:at + n].to(DEV)
+        outs.append(kernels.linear_scan(rows[:, :a], rows[:, a:2 * a], rows[:, 2 * a:], state, _i64([1]), _i32([0, n]), H, dk, dv,
+                                        head_decay=decay.to(DEV), k_scale=0.25, silu=silu, q_lens=[n], plan_cache={}).cpu())
+        at += n
+    got = torch.cat(outs).double()
+    tol = 3e-3 if silu else 3e-5            # (silu: the single token's walk does not round it, and the hardware's last bits move roundings)
+    assert (got - want).abs().max() < tol * want.abs().max()
+    assert (state[1].cpu().double() - S).abs().max() < tol * S.abs().max()
+    assert float(state[0].abs().max()) == 0
 
 
 def test_rows_normed_together_and_gated():

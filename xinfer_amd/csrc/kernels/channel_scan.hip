@@ -23,12 +23,23 @@ namespace xi {
 
 constexpr int kScanAhead = 8;
 
-static __device__ __forceinline__ float sigmoid_f(float x) { return 1.f / (1.f + expf(-x)); }
+constexpr float kLog2eC = 1.4426950408889634f;
+
+// FAST (the bfloat16 path): the hardware's exponential, reciprocal and square root, each within an ulp of float32; the
+// 32-bit path takes the library's.
+template <bool FAST> static __device__ __forceinline__ float exp_f(float x) {
+  return FAST ? __builtin_amdgcn_exp2f(x * kLog2eC) : expf(x);
+}
+template <bool FAST> static __device__ __forceinline__ float inv_f(float x) { return FAST ? __builtin_amdgcn_rcpf(x) : 1.f / x; }
+template <bool FAST> static __device__ __forceinline__ float sigmoid_f(float x) { return inv_f<FAST>(1.f + exp_f<FAST>(-x)); }
 
 // act 0: none, 1: silu, 2: the tanh form of gelu
-static __device__ __forceinline__ float gate_of(float g, int act) {
-  if (act == 1) return g / (1.f + expf(-g));
-  if (act == 2) return 0.5f * g * (1.f + tanhf(0.7978845608028654f * (g + 0.044715f * g * g * g)));
+template <bool FAST> static __device__ __forceinline__ float gate_of(float g, int act) {
+  if (act == 1) return g * sigmoid_f<FAST>(g);
+  if (act == 2) {          // 1 + tanh(y) = 2 sigmoid(2 y)
+    const float y = 0.7978845608028654f * (g + 0.044715f * g * g * g);
+    return FAST ? g * sigmoid_f<FAST>(2.f * y) : 0.5f * g * (1.f + tanhf(y));
+  }
   return g;
 }
 
@@ -94,15 +105,16 @@ static __device__ __forceinline__ void operands(const ChannelArgs& A, int t, int
     load_run<V>(A.b + (size_t)t * A.C + c, q);
   }
 }
-template <bool MIN, int V>
+template <bool FAST, bool MIN, int V>
 static __device__ __forceinline__ void make_terms(float (&p)[V], float (&q)[V], const float (&zb)[V], const float (&ub)[V]) {
   if constexpr (MIN) {
 #pragma unroll
     for (int i = 0; i < V; ++i) {
       const float z = p[i] + zb[i], u = q[i] + ub[i];
-      const float cand = u >= 0.f ? u + 0.5f : sigmoid_f(u);
-      p[i] = sigmoid_f(-z);                 // 1 - sigmoid(z)
-      q[i] = sigmoid_f(z) * cand;
+      const float cand = u >= 0.f ? u + 0.5f : sigmoid_f<FAST>(u);
+      const float e = exp_f<FAST>(-fabsf(z)), big = inv_f<FAST>(1.f + e), small = e * big;      // sigmoid(|z|), sigmoid(-|z|)
+      p[i] = z >= 0.f ? small : big;          // 1 - sigmoid(z)
+      q[i] = (z >= 0.f ? big : small) * cand;
     }
   }
 }
@@ -144,7 +156,7 @@ __global__ __launch_bounds__(256) void channel_share_kernel(const ChannelArgs A)
 #pragma unroll
     for (int k = 0; k < kScanAhead; ++k) {
       if (t0 + k >= it.last) break;
-      make_terms<MIN, V>(p[k], q[k], zb, ub);
+      make_terms<sizeof(T) == 2, MIN, V>(p[k], q[k], zb, ub);
 #pragma unroll
       for (int i = 0; i < V; ++i) {
         pa[i] *= p[k][i];
@@ -204,12 +216,12 @@ __global__ __launch_bounds__(256) void channel_walk_kernel(const ChannelArgs A) 
 #pragma unroll
     for (int k = 0; k < kScanAhead; ++k) {
       if (t0 + k >= it.last) break;
-      make_terms<MIN, V>(p[k], q[k], zb, ub);
+      make_terms<sizeof(T) == 2, MIN, V>(p[k], q[k], zb, ub);
       float o[V];
 #pragma unroll
       for (int i = 0; i < V; ++i) {
         s[i] = fmaf(p[k][i], s[i], q[k][i]);
-        o[i] = s[i] * gate_of(gv[k][i] + gb[i], A.act);
+        o[i] = s[i] * gate_of<sizeof(T) == 2>(gv[k][i] + gb[i], A.act);
       }
       store_run<V>(out + (size_t)(t0 + k) * A.C + c, o);
     }
@@ -218,10 +230,19 @@ __global__ __launch_bounds__(256) void channel_walk_kernel(const ChannelArgs A) 
 }
 
 // ---- the real-gated linear recurrent unit's a and b ------------------------------------------------------------
+template <bool FAST>
 static __device__ __forceinline__ void rglru_ab(float r_logit, float i_logit, float rate, float u, float& a, float& b) {
-  const float log_a = rate * sigmoid_f(r_logit);
-  a = expf(log_a);
-  b = sqrtf(-expm1f(2.f * log_a)) * sigmoid_f(i_logit) * u;
+  const float log_a = rate * sigmoid_f<FAST>(r_logit);
+  a = exp_f<FAST>(log_a);
+  const float x = 2.f * log_a;               // 1 - a^2 = 1 - e^x, x <= 0
+  if (FAST) {
+    // near 0 by the series of e^x - 1 (x^8 / 8! is below a float32 ulp of it for |x| < 0.35)
+    const float series = -x * fmaf(x * 0.5f, fmaf(x * (1.f / 3.f), fmaf(x * 0.25f, fmaf(x * 0.2f, fmaf(x * (1.f / 6.f), fmaf(x, 1.f / 7.f, 1.f), 1.f), 1.f), 1.f), 1.f), 1.f);
+    const float rest = x > -0.35f ? series : 1.f - exp_f<true>(x);
+    b = __builtin_amdgcn_sqrtf(rest) * sigmoid_f<true>(i_logit) * u;
+  } else {
+    b = sqrtf(-expm1f(x)) * sigmoid_f<false>(i_logit) * u;
+  }
 }
 
 // logits float32 [T, blocks, 2, per]: a block's r part, then its i part
@@ -235,7 +256,7 @@ __global__ __launch_bounds__(256) void rglru_terms_kernel(const float* __restric
     const int c = (int)(e - t * C);
     const int blk = c / per, k = c - blk * per;
     const float* l = logits + (size_t)t * 2 * C + (size_t)blk * 2 * per + k;
-    rglru_ab(l[0] + r_bias[c], l[per] + i_bias[c], rate[c], to_float(u[e]), a[e], b[e]);
+    rglru_ab<false>(l[0] + r_bias[c], l[per] + i_bias[c], rate[c], to_float(u[e]), a[e], b[e]);
   }
 }
 
@@ -313,7 +334,7 @@ __global__ __launch_bounds__(256) void rglru_gates_kernel(const bf16* __restrict
       float a4[4], b4[4];
 #pragma unroll
       for (int i = 0; i < 4; ++i)
-        rglru_ab(acc[ti][tj][i] + r_bias[c + i], acc[ti + 2][tj][i] + i_bias[c + i], rate[c + i], u4[i], a4[i], b4[i]);
+        rglru_ab<true>(acc[ti][tj][i] + r_bias[c + i], acc[ti + 2][tj][i] + i_bias[c + i], rate[c + i], u4[i], a4[i], b4[i]);
       *reinterpret_cast<float4*>(a_out + (size_t)t * C + c) = make_float4(a4[0], a4[1], a4[2], a4[3]);
       *reinterpret_cast<float4*>(b_out + (size_t)t * C + c) = make_float4(b4[0], b4[1], b4[2], b4[3]);
     }

@@ -376,8 +376,14 @@ __global__ __launch_bounds__(1024) void qk_norm_rope_kvt_bf16_kernel(
   {
     bf16x8v x;
     if (on) x = *reinterpret_cast<const bf16x8v*>(qkv + ((size_t)t * heads + h) * d + 8 * c);
+    float bv[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+    if (bias) {
+      const float4* bp = reinterpret_cast<const float4*>(bias + (size_t)h * d + 8 * c);
+      const float4 b0 = bp[0], b1 = bp[1];
+      bv[0] = b0.x; bv[1] = b0.y; bv[2] = b0.z; bv[3] = b0.w; bv[4] = b1.x; bv[5] = b1.y; bv[6] = b1.z; bv[7] = b1.w;
+    }
 #pragma unroll
-    for (int e = 0; e < 8; ++e) v[e] = on ? to_float(x.v[e]) + (bias ? bias[(size_t)h * d + 8 * c + e] : 0.f) : 0.f;
+    for (int e = 0; e < 8; ++e) v[e] = on ? to_float(x.v[e]) + bv[e] : 0.f;
   }
   const float* w = is_k ? kw : qw;
   if (w) {
@@ -403,7 +409,20 @@ __global__ __launch_bounds__(1024) void qk_norm_rope_kvt_bf16_kernel(
   const int half = rot >> 1;
   const int pos = positions[t < n_tok ? t : n_tok - 1];
   float o[8];
-  if (interleaved) {
+  if (interleaved && rot % 8 == 0) {       // a lane's 8 elements turn together or not at all: its 4 pairs' angles in two loads
+    const bool in_rot = 8 * c < rot;
+    float4 cs = float4{1.f, 1.f, 1.f, 1.f}, sn = float4{0.f, 0.f, 0.f, 0.f};
+    if (in_rot) {
+      cs = *reinterpret_cast<const float4*>(cos_t + (size_t)pos * half + 4 * c);
+      sn = *reinterpret_cast<const float4*>(sin_t + (size_t)pos * half + 4 * c);
+    }
+    const float c4[4] = {cs.x, cs.y, cs.z, cs.w}, s4[4] = {sn.x, sn.y, sn.z, sn.w};
+#pragma unroll
+    for (int e = 0; e < 8; e += 2) {
+      o[e] = in_rot ? v[e] * c4[e / 2] - v[e + 1] * s4[e / 2] : v[e];
+      o[e + 1] = in_rot ? v[e] * s4[e / 2] + v[e + 1] * c4[e / 2] : v[e + 1];
+    }
+  } else if (interleaved) {
 #pragma unroll
     for (int e = 0; e < 8; e += 2) {
       const int i = 8 * c + e;

@@ -243,6 +243,31 @@ __global__ __launch_bounds__(256) void embed_norm_kernel(const T* __restrict__ t
   for (int i = threadIdx.x; i < H; i += 256) o[i] = to_float(row[i]) * scale * inv * w[i];
 }
 
+// Rows of a multiple of 4 elements, up to 4 NT MAXV, kept in registers between the sum and the store.
+template <typename T, int NT, int MAXV>
+__global__ __launch_bounds__(NT) void embed_norm_vec_kernel(const T* __restrict__ table, const int* __restrict__ ids, float scale,
+                                                            const float* __restrict__ w, float eps, float* __restrict__ out, int H) {
+  __shared__ float scratch[NT / kWave];
+  const T* row = table + (size_t)ids[blockIdx.x] * H;
+  float* o = out + (size_t)blockIdx.x * H;
+  const int nvec = H / 4;
+  float4 x[MAXV];
+  float ss = 0.f;
+#pragma unroll
+  for (int v = 0; v < MAXV; ++v) {
+    const int i = v * NT + threadIdx.x;
+    x[v] = i < nvec ? join_load4(row + 4 * i) : float4{0.f, 0.f, 0.f, 0.f};
+    x[v] = float4{x[v].x * scale, x[v].y * scale, x[v].z * scale, x[v].w * scale};
+    ss += dot4(x[v]);
+  }
+  const float inv = rsqrtf(block_sum<NT / kWave>(ss, scratch) / (float)H + eps);
+#pragma unroll
+  for (int v = 0; v < MAXV; ++v) {
+    const int i = v * NT + threadIdx.x;
+    if (i < nvec) join_store4(o + 4 * i, mul4(x[v], inv, join_load4(w + 4 * i)));
+  }
+}
+
 template <typename TO>
 static void launch_join(const JoinArgs& A, int n, hipStream_t stream, bool aligned) {
   const int H = A.H;
@@ -351,10 +376,24 @@ int xi_stream_join(const float* x, int n_terms, const void* const* y, const int*
 int xi_embed_norm(const void* table, int dtype, const int* ids, float scale, const float* w, float eps, float* out, int n_tok, int H,
                   hipStream_t stream) {
   XI_CHECK(n_tok >= 0 && H > 0 && w, "embed_norm: bad sizes T=%d H=%d", n_tok, H);
+  XI_CHECK(dtype == kF32 || dtype == kBF16, "embed_norm: unknown dtype %d", dtype);
   if (n_tok == 0) return 0;
+  if (H % 4 == 0 && H <= 8192 && ((reinterpret_cast<uintptr_t>(table) | reinterpret_cast<uintptr_t>(w) | reinterpret_cast<uintptr_t>(out)) & 15) == 0) {
+#define XI_EN(NT, MAXV)                                                                                                                  \
+  do {                                                                                                                                   \
+    if (dtype == kF32) embed_norm_vec_kernel<float, NT, MAXV><<<n_tok, NT, 0, stream>>>((const float*)table, ids, scale, w, eps, out, H); \
+    else embed_norm_vec_kernel<bf16, NT, MAXV><<<n_tok, NT, 0, stream>>>((const bf16*)table, ids, scale, w, eps, out, H);                \
+  } while (0)
+    if (H <= 1024) XI_EN(256, 1);
+    else if (n_tok <= 256) XI_EN(1024, 2);
+    else if (H <= 4096) XI_EN(256, 4);
+    else XI_EN(512, 4);
+#undef XI_EN
+    XI_LAUNCH_CHECK("embed_norm");
+    return 0;
+  }
   if (dtype == kF32) embed_norm_kernel<float><<<n_tok, 256, 0, stream>>>((const float*)table, ids, scale, w, eps, out, H);
-  else if (dtype == kBF16) embed_norm_kernel<bf16><<<n_tok, 256, 0, stream>>>((const bf16*)table, ids, scale, w, eps, out, H);
-  else XI_CHECK(false, "embed_norm: unknown dtype %d", dtype);
+  else embed_norm_kernel<bf16><<<n_tok, 256, 0, stream>>>((const bf16*)table, ids, scale, w, eps, out, H);
   XI_LAUNCH_CHECK("embed_norm");
   return 0;
 }

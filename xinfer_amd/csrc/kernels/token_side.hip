@@ -1,7 +1,7 @@
 // A layer's own input for the token: g[t, d] = gelu_tanh(z[t, d]) * e[ids[t], offset + d], z = W x, e a table row's part
 // that belongs to the layer.  `side_mul_kernel` takes z as a product left it (rows, or a stack of float32 partial sums);
-// `side_gate_kernel` makes z itself in steps of few tokens: a wave owns one output d and takes up to kSideTok tokens at
-// a time, so that a row of W is read once for all of them.  Float32 until the one rounding of g.
+// `side_gate_kernel` makes z itself in steps of few tokens: a workgroup owns one output d, its waves a part of K each, and
+// takes up to kSideTok tokens at a time, so that a row of W is read once for all of them.  Float32 until the one rounding of g.
 #include "common.h"
 
 namespace xi {
@@ -29,19 +29,19 @@ __global__ __launch_bounds__(256) void side_mul_kernel(const void* __restrict__ 
   }
 }
 
-constexpr int kSideTok = 8;
+constexpr int kSideTok = 8, kSideWaves = 4;
 
 // K a multiple of 8, bfloat16
-__global__ __launch_bounds__(256) void side_gate_kernel(const bf16* __restrict__ x, const bf16* __restrict__ w,
+__global__ __launch_bounds__(kSideWaves* kWave) void side_gate_kernel(const bf16* __restrict__ x, const bf16* __restrict__ w,
                                                         const bf16* __restrict__ table, long long row_len, int offset,
                                                         const int* __restrict__ ids, bf16* __restrict__ out, int n_tok, int dim, int K) {
-  const int d = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
-  if (d >= dim) return;
+  __shared__ float part[kSideWaves][kSideTok];
+  const int d = blockIdx.x, wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int t0 = blockIdx.y * kSideTok;
   float acc[kSideTok];
 #pragma unroll
   for (int t = 0; t < kSideTok; ++t) acc[t] = 0.f;
-  for (int k = 8 * lane; k < K; k += 8 * kWave) {
+  for (int k = 8 * threadIdx.x; k < K; k += 8 * kSideWaves * kWave) {
     const uint4 wr = *reinterpret_cast<const uint4*>(w + (size_t)d * K + k);
     const unsigned wu[4] = {wr.x, wr.y, wr.z, wr.w};
     uint4 xr[kSideTok];
@@ -63,8 +63,13 @@ __global__ __launch_bounds__(256) void side_gate_kernel(const bf16* __restrict__
 #pragma unroll
   for (int t = 0; t < kSideTok; ++t) {
     const float z = wave_sum(acc[t]);
-    if (lane == t && t0 + t < n_tok)
-      out[(size_t)(t0 + t) * dim + d] = from_float<bf16>(side_gelu(z) * to_float(table[(size_t)ids[t0 + t] * row_len + offset + d]));
+    if (lane == 0) part[wave][t] = z;
+  }
+  __syncthreads();
+  const int t = threadIdx.x;
+  if (t < kSideTok && t0 + t < n_tok) {
+    const float z = (part[0][t] + part[1][t]) + (part[2][t] + part[3][t]);
+    out[(size_t)(t0 + t) * dim + d] = from_float<bf16>(side_gelu(z) * to_float(table[(size_t)ids[t0 + t] * row_len + offset + d]));
   }
 }
 
@@ -102,9 +107,9 @@ int xi_side_gate(const void* x, const void* w, const void* table, long long row_
            "side_gate: bad sizes T=%d dim=%d K=%d offset=%d", n_tok, dim, K, offset);
   XI_CHECK((reinterpret_cast<uintptr_t>(x) & 15) == 0 && (reinterpret_cast<uintptr_t>(w) & 15) == 0, "side_gate: rows in whole 16-byte chunks");
   if (n_tok == 0) return 0;
-  dim3 grid((unsigned)((dim + 3) / 4), (unsigned)((n_tok + kSideTok - 1) / kSideTok));
+  dim3 grid((unsigned)dim, (unsigned)((n_tok + kSideTok - 1) / kSideTok));
   XI_CHECK(grid.y <= 65535u, "side_gate: too many tokens");
-  side_gate_kernel<<<grid, 256, 0, stream>>>((const bf16*)x, (const bf16*)w, (const bf16*)table, row_len, offset, ids, (bf16*)out, n_tok,
+  side_gate_kernel<<<grid, kSideWaves * kWave, 0, stream>>>((const bf16*)x, (const bf16*)w, (const bf16*)table, row_len, offset, ids, (bf16*)out, n_tok,
                                              dim, K);
   XI_LAUNCH_CHECK("side_gate");
   return 0;

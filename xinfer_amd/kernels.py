@@ -277,6 +277,68 @@ def scan_chunk_plan(q_lens, chunk: Optional[int] = None):
     return whole, long, chunks
 
 
+DECAY_MFMA = True                 # False: portions under one constant decay a head go through the walk token by token too
+DECAY_CHUNK = 64                  # tokens of a chunk of `xi_decay_chunks` at most
+DECAY_FROM = 32                   # tokens of a portion from which it is cut into such chunks
+DECAY_BYTES_MOST = 4 << 30        # the chunks' states are kept side by side: steps that would need more go through the walk
+
+
+def decay_chunk_plan(q_lens, chunk: int = DECAY_CHUNK):
+    """The portions of a step for `xi_decay_chunks`: (whole, long, chunks) as `scan_chunk_plan` gives them, portions from
+    DECAY_FROM tokens on cut into chunks of `chunk` tokens."""
+    whole, long, chunks = [], [], []
+    for b, n in enumerate(q_lens):
+        n = int(n)
+        if n < DECAY_FROM:
+            whole.append(b)
+            continue
+        long.append((b, len(chunks), -(-n // chunk)))
+        chunks += [(c, min(chunk, n - c)) for c in range(0, n, chunk)]
+    return whole, long, chunks
+
+
+def _decay_chunks(common, state, slot_stride, state_slots, q_lens, plan_cache, out, H, dk, dv, q_scale, k_scale) -> bool:
+    """`linear_scan` for a step with long portions in bfloat16 under one decay a head: the long ones on the matrix cores, the
+    others in one piece.  False: nothing was done (sizes, rows or lengths that it does not take)."""
+    q, k, v, qs, ks, vs, head_decay, silu = common[0], common[1], common[2], common[3], common[4], common[5], common[9], common[17]
+    if (not DECAY_MFMA or SCAN_CHUNK <= 0 or q.dtype != torch.bfloat16 or head_decay is None or common[15] != dv or common[16] != 1
+            or not lib().xi_decay_chunks_takes(dk, dv) or qs % 8 or ks % 8 or vs % 8
+            or any(t.data_ptr() % 16 for t in (q, k, v))):
+        return False
+    chunk = min(DECAY_CHUNK, SCAN_CHUNK)
+    key = ("decay_chunk_plan", chunk, DECAY_FROM)
+    plan = plan_cache.get(key) if plan_cache is not None else None
+    if plan is None:
+        whole, long, chunks = decay_chunk_plan(q_lens, chunk)
+        starts = [0]
+        for n in q_lens:
+            starts.append(starts[-1] + int(n))
+        C, L, W = len(chunks), len(long), len(whole)
+        first = [0] * C
+        for b, c0, count in long:
+            for c in range(c0, c0 + count):
+                first[c] = starts[b] + chunks[c][0]
+        i32 = torch.tensor(first + [f + n for f, (_, n) in zip(first, chunks)] + [c0 for _, c0, _ in long] + [n for _, _, n in long]
+                           + [starts[b] for b in whole] + [starts[b + 1] for b in whole], dtype=torch.int32).to(q.device)
+        i64 = torch.tensor([b for b, _, _ in long] + whole, dtype=torch.int64).to(q.device)
+        slots = state_slots.index_select(0, i64)
+        plan = dict(C=C, L=L, W=W, first=i32[:C], last=i32[C:2 * C], c0=i32[2 * C:2 * C + L], n=i32[2 * C + L:2 * C + 2 * L],
+                    wfirst=i32[2 * C + 2 * L:2 * C + 2 * L + W], wlast=i32[2 * C + 2 * L + W:], long_slots=slots[:L], whole_slots=slots[L:])
+        if plan_cache is not None:
+            plan_cache[key] = plan
+    if not plan["L"] or plan["C"] * H * dk * dv * 4 > DECAY_BYTES_MOST:
+        return False
+    ll, P = ctypes.c_longlong, plan
+    shares = torch.empty((P["C"], H, dk, dv), dtype=torch.float32, device=q.device)
+    _ok(lib().xi_decay_chunks(_p(q), ll(qs), _p(k), ll(ks), _p(v), ll(vs), _p(head_decay), _p(state), ll(slot_stride), _p(P["long_slots"]),
+                              _p(P["c0"]), _p(P["n"]), P["L"], _p(P["first"]), _p(P["last"]), P["C"], _p(shares), _p(out), H, dk, dv,
+                              ctypes.c_float(q_scale), ctypes.c_float(k_scale), int(silu), _stream()))
+    if P["W"]:
+        _scan_launch(*common, state, slot_stride, P["whole_slots"], state, slot_stride, P["whole_slots"], P["wfirst"].data_ptr(),
+                     P["wlast"].data_ptr(), out, None, P["W"], H, dk, dv, q_scale, k_scale)
+    return True
+
+
 def _scan_launch(q, k, v, qs, ks, vs, z, z_bias, tau, head_decay, step, ss, step_bias, decay_log, gates, v_cols, group_heads, act,
                  state_in, in_stride, in_idx, state_out, out_stride, out_idx,
                  first, last, out, decay_out, items, H, dk, dv, q_scale, k_scale):
@@ -312,7 +374,8 @@ def linear_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: torch.
     `q_lens` (the host's copy of the portions' lengths; None: nothing of the step is read on the host, as a step
     of single tokens wants it): portions of two chunks and more (`SCAN_CHUNK`) are cut into chunks that are walked
     side by side in three launches (each chunk's own share from a zero state; the states the chunks start from,
-    one after the other; the chunks' results), the others in one piece.  `plan_cache`: a dict of the step in which
+    one after the other; the chunks' results), the others in one piece; in bfloat16 with a constant decay per head the long
+    ones go through the matrix cores (`xi_decay_chunks`, portions from DECAY_FROM tokens on).  `plan_cache`: a dict of the step in which
     the index arrays of this cutting are kept for the next layer."""
     H, dk, dv = int(heads), int(key_dim), int(value_dim)
     T = q.shape[0]
@@ -371,6 +434,8 @@ def linear_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: torch.
     out = torch.empty((T, H, dv), dtype=torch.float32, device=q.device)
     slot_stride = int(state.stride(0)) if state.shape[0] > 1 else H * dk * dv
     common = (q, k, v, qs, ks, vs, z, z_bias, tau, head_decay, step, ss, step_bias, decay_log, gates, vc, H // G, int(bool(silu)))
+    if q_lens is not None and _decay_chunks(common, state, slot_stride, state_slots, q_lens, plan_cache, out, H, dk, dv, q_scale, k_scale):
+        return out
     whole, long, chunks = scan_chunk_plan(q_lens) if q_lens is not None else (None, [], [])
     if not long:            # every request in one piece, straight from the step's own arrays
         _scan_launch(*common, state, slot_stride, state_slots, state, slot_stride, state_slots, cu_q.data_ptr(),
