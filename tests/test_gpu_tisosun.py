@@ -380,12 +380,14 @@ def _read_pools(k_pool, v_pool, table, L, grouped):
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("H,G,d,dv,rot,page,norms", [(6, 2, 16, 24, 8, 16, True), (5, 5, 20, 12, 20, 8, True), (3, 1, 12, 20, 6, 8, True),
+@pytest.mark.parametrize("L", [45, 301])
+@pytest.mark.parametrize("H,G,d,dv,rot,page,norms", [(6, 2, 16, 24, 8, 16, True), (2, 2, 128, 40, 64, 16, True), (3, 1, 24, 256, 12, 8, True), (5, 5, 20, 12, 20, 8, True), (3, 1, 12, 20, 6, 8, True),
                                                      (2, 1, 10, 6, 0, 8, True), (4, 2, 64, 48, 32, 64, True), (3, 3, 16, 8, 16, 8, False)])
-def test_heads_with_biases_norms_and_turned_pairs(H, G, d, dv, rot, page, norms, dtype):
-    """Bias, norm with a weight, rotation of the pairs (2i, 2i + 1) in that order, and the cache write."""
+def test_heads_with_biases_norms_and_turned_pairs(H, G, d, dv, rot, page, norms, L, dtype):
+    """Bias, norm with a weight, rotation of the pairs (2i, 2i + 1) in that order, and the cache write, a head a wave and (many
+    tokens, sizes in eights) eight dims a lane."""
     from xinfer_amd import kernels
-    dt, eps, L = TD[dtype], 1e-5, 45
+    dt, eps = TD[dtype], 1e-5
     grouped = dtype == "bfloat16"
     g = torch.Generator().manual_seed(H * 10 + d)
     width = (H + G) * d + G * dv

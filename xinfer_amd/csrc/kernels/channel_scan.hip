@@ -21,7 +21,8 @@
 
 namespace xi {
 
-constexpr int kScanAhead = 8;
+constexpr int kScanAhead = 8;       // tokens whose operands are asked for at once
+constexpr int kShareAhead = 16;     // chunks whose shares are
 
 constexpr float kLog2eC = 1.4426950408889634f;
 
@@ -185,16 +186,16 @@ __global__ __launch_bounds__(256) void channel_walk_kernel(const ChannelArgs A) 
   }
   if (it.count > 1) {
     load_run<V>(A.init + (size_t)it.lead * A.C + c, s);
-    for (int j0 = it.lead; j0 < n; j0 += 4) {           // the chunks before this one, in order, four asked for at once
-      float pa[4][V], sum[4][V];
+    for (int j0 = it.lead; j0 < n; j0 += kShareAhead) {           // the chunks before this one, in order
+      float pa[kShareAhead][V], sum[kShareAhead][V];
 #pragma unroll
-      for (int k = 0; k < 4; ++k) {
+      for (int k = 0; k < kShareAhead; ++k) {
         const size_t at = (size_t)(j0 + k < n ? j0 + k : n - 1) * 2 * A.C + c;
         load_run<V>(A.share + at, pa[k]);
         load_run<V>(A.share + at + A.C, sum[k]);
       }
 #pragma unroll
-      for (int k = 0; k < 4; ++k) {
+      for (int k = 0; k < kShareAhead; ++k) {
         if (j0 + k >= n) break;
 #pragma unroll
         for (int i = 0; i < V; ++i) s[i] = fmaf(pa[k][i], s[i], sum[k][i]);

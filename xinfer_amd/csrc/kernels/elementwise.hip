@@ -306,8 +306,8 @@ __global__ void qk_norm_rope_kv_kernel(const void* __restrict__ qkv_v, int slice
 // group of lanes), a wave holds 64/(d/8) tokens, the workgroup's waves hold the block.  The
 // workgroup of a V head turns its [tokens, d] tile through LDS so that a wave's store takes eight
 // tokens by eight dims: where the eight tokens follow each other in a group of the pool, one line
-// of 128 bytes.
-// Needs d % 8 == 0 and, for the half layout, rotary_dim % 16 == 0 (the partner of a lane's
+// of 128 bytes.  Value heads may have a size of their own, dv.
+// Needs d % 8 == 0, dv % 8 == 0 and, for the half layout, rotary_dim % 16 == 0 (the partner of a lane's
 // 8 elements is then another lane's 8 elements).
 struct alignas(16) bf16x8v { bf16 v[8]; };
 
@@ -315,10 +315,10 @@ __global__ __launch_bounds__(1024) void qk_norm_rope_kvt_bf16_kernel(
     const bf16* __restrict__ qkv, const float* __restrict__ bias, const float* __restrict__ qw, const float* __restrict__ kw, float eps,
     const float* __restrict__ cos_t, const float* __restrict__ sin_t, int rot, int interleaved,
     const int* __restrict__ positions, const long long* __restrict__ slots, bf16* __restrict__ q_out,
-    bf16* __restrict__ k_cache, bf16* __restrict__ vt_cache, int page_size, int n_tok, int nq, int nkv, int d) {
+    bf16* __restrict__ k_cache, bf16* __restrict__ vt_cache, int page_size, int n_tok, int nq, int nkv, int d, int dv) {
   extern __shared__ __align__(16) unsigned char smem_raw[];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
-  const int heads = nq + 2 * nkv;
+  const size_t width = (size_t)(nq + nkv) * d + (size_t)nkv * dv;      // of a packed row
   const int lph = d >> 3;          // lanes per head
   const int hpw = 64 / lph;        // tokens a wave holds
   const int tpw = (blockDim.x >> 6) * hpw;   // tokens of the workgroup (at most 64)
@@ -332,8 +332,8 @@ __global__ __launch_bounds__(1024) void qk_norm_rope_kvt_bf16_kernel(
   if (h >= nq + nkv) {
     // ---- a V head: tile into LDS, then lanes along the token axis
     const int kvh = h - nq - nkv;
-    bf16* vs = reinterpret_cast<bf16*>(smem_raw);  // [tpw][d + 2]
-    const int vstride = d + 2;                      // an odd number of 32-bit words per row
+    bf16* vs = reinterpret_cast<bf16*>(smem_raw);  // [tpw][dv + 2]
+    const int vstride = dv + 2;                      // an odd number of 32-bit words per row
     // Every lane looks up where its own token of the block goes (lane = token); a store then takes eight
     // tokens by eight dims: lane -> token 8 tg + (lane & 7), dim i0 + (lane >> 3), the place handed over
     // from the token's lane.
@@ -342,26 +342,29 @@ __global__ __launch_bounds__(1024) void qk_norm_rope_kvt_bf16_kernel(
     if (slot >= 0) {
       const long long page = slot / page_size;
       const int off = (int)(slot - page * page_size);
-      place = ((unsigned long long)page * nkv + kvh) * d * page_size + (unsigned long long)(off >> 3) * d * 8 + (off & 7);
+      place = ((unsigned long long)page * nkv + kvh) * dv * page_size + (unsigned long long)(off >> 3) * dv * 8 + (off & 7);
     }
-    if (on) {
-      uint4 raw = *reinterpret_cast<const uint4*>(qkv + ((size_t)t * heads + h) * d + 8 * c);
+    const size_t col0 = (size_t)(nq + nkv) * d + (size_t)kvh * dv;
+    for (int u = tid; u < tpw * (dv >> 3); u += (int)blockDim.x) {
+      const int tok = u / (dv >> 3), cc = 8 * (u - tok * (dv >> 3));
+      if (t0 + tok >= n_tok) break;
+      uint4 raw = *reinterpret_cast<const uint4*>(qkv + (size_t)(t0 + tok) * width + col0 + cc);
       if (bias) {
         bf16x8v x = *reinterpret_cast<const bf16x8v*>(&raw);
 #pragma unroll
-        for (int e = 0; e < 8; ++e) x.v[e] = from_float<bf16>(to_float(x.v[e]) + bias[(size_t)h * d + 8 * c + e]);
+        for (int e = 0; e < 8; ++e) x.v[e] = from_float<bf16>(to_float(x.v[e]) + bias[col0 + cc + e]);
         raw = *reinterpret_cast<const uint4*>(&x);
       }
-      unsigned* dst = reinterpret_cast<unsigned*>(vs + tl * vstride + 8 * c);
+      unsigned* dst = reinterpret_cast<unsigned*>(vs + tok * vstride + cc);
       dst[0] = raw.x;
       dst[1] = raw.y;
       dst[2] = raw.z;
       dst[3] = raw.w;
     }
     __syncthreads();
-    const int units = ((tpw + 7) >> 3) * (d >> 3);
+    const int units = ((tpw + 7) >> 3) * (dv >> 3);
     for (int u = wave; u < units; u += (int)(blockDim.x >> 6)) {
-      const int tg = u / (d >> 3), i = 8 * (u - tg * (d >> 3)) + (lane >> 3);
+      const int tg = u / (dv >> 3), i = 8 * (u - tg * (dv >> 3)) + (lane >> 3);
       const int tok = 8 * tg + (lane & 7);
       const unsigned lo = __shfl((unsigned)place, tok, kWave), hi = __shfl((unsigned)(place >> 32), tok, kWave);
       const unsigned long long at = ((unsigned long long)hi << 32) | lo;
@@ -375,7 +378,7 @@ __global__ __launch_bounds__(1024) void qk_norm_rope_kvt_bf16_kernel(
   float v[8];
   {
     bf16x8v x;
-    if (on) x = *reinterpret_cast<const bf16x8v*>(qkv + ((size_t)t * heads + h) * d + 8 * c);
+    if (on) x = *reinterpret_cast<const bf16x8v*>(qkv + (size_t)t * width + (size_t)h * d + 8 * c);
     float bv[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
     if (bias) {
       const float4* bp = reinterpret_cast<const float4*>(bias + (size_t)h * d + 8 * c);
@@ -1025,11 +1028,12 @@ int xi_silu_mul(const void* gate_up, void* out, int dtype, int n_tok, int I, hip
 }
 
 // qkv: [T, heads * d] in `dtype`, or, with slices > 0, float32 partial sums [slices, T, heads * d]
-// of it (then `dtype` is that of q_out and the cache, and the form of one wave per head runs).
+// of it (then `dtype` is that of q_out and the cache, and the form of one wave per head runs).  dv: the value heads' size;
+// one that is not d is for the vectorized form alone (bfloat16, V in groups of eight keys, sizes in eights).
 int xi_qk_norm_rope_kv(const void* qkv, int dtype, int slices, const float* bias, const float* qw, const float* kw, float eps,
                        const float* cos_t, const float* sin_t, int rot, int interleaved,
                        const int* positions, const long long* slots, void* q_out, void* k_cache,
-                       void* v_cache, int page_size, int n_tok, int nq, int nkv, int d, int v_grouped,
+                       void* v_cache, int page_size, int n_tok, int nq, int nkv, int d, int dv, int v_grouped,
                        int vector_min_tokens, hipStream_t stream) {
   XI_CHECK(n_tok >= 0 && nq > 0 && nkv > 0 && d > 0 && page_size > 0,
            "qk_norm_rope_kv: bad sizes T=%d nq=%d nkv=%d d=%d page=%d", n_tok, nq, nkv, d, page_size);
@@ -1043,6 +1047,7 @@ int xi_qk_norm_rope_kv(const void* qkv, int dtype, int slices, const float* bias
   XI_CHECK(!v_grouped || page_size % 8 == 0, "qk_norm_rope_kv: V in groups of eight keys needs pages of a multiple of 8 tokens, not %d",
            page_size);
   if (slices == 0 && n_tok >= vector_min_tokens && dtype == kBF16 && v_grouped && d % 8 == 0 && d <= 256 &&
+      dv % 8 == 0 && dv > 0 && dv <= 256 &&
       (interleaved || rot % 16 == 0) &&
       ((uintptr_t)qkv | (uintptr_t)q_out | (uintptr_t)k_cache | (uintptr_t)cos_t | (uintptr_t)sin_t) % 16 == 0) {
     const int lph = d / 8, hpw = 64 / lph;
@@ -1051,13 +1056,14 @@ int xi_qk_norm_rope_kv(const void* qkv, int dtype, int slices, const float* bias
     const int tpw = n_waves * hpw;
     const unsigned blocks_x = (unsigned)((n_tok + tpw - 1) / tpw);
     XI_CHECK(nq + 2 * nkv <= 65535, "qk_norm_rope_kv: too many heads");
-    const size_t lds = (size_t)tpw * (d + 2) * sizeof(bf16);
+    const size_t lds = (size_t)tpw * (dv + 2) * sizeof(bf16);
     qk_norm_rope_kvt_bf16_kernel<<<dim3(blocks_x, nq + 2 * nkv), n_waves * 64, lds, stream>>>(
         (const bf16*)qkv, bias, qw, kw, eps, cos_t, sin_t, rot, interleaved, positions, slots, (bf16*)q_out,
-        (bf16*)k_cache, (bf16*)v_cache, page_size, n_tok, nq, nkv, d);
+        (bf16*)k_cache, (bf16*)v_cache, page_size, n_tok, nq, nkv, d, dv);
     XI_LAUNCH_CHECK("qk_norm_rope_kv");
     return 0;
   }
+  XI_CHECK(dv == d, "qk_norm_rope_kv: value heads of %d beside keys of %d need the vectorized form", dv, d);
   const long long waves = (long long)n_tok * (nq + 2 * nkv);
   const int wpb = 4;
   const long long blocks = (waves + wpb - 1) / wpb;

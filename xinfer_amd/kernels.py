@@ -842,7 +842,7 @@ def qk_norm_rope_kv(qkv: torch.Tensor, q_weight: Optional[torch.Tensor],
     _ok(lib().xi_qk_norm_rope_kv(
         _p(qkv), _code(q_out, "qk_norm_rope_kv"), slices, _p(bias), _p(q_weight), _p(k_weight), ctypes.c_float(eps),
         _p(cos), _p(sin), int(rotary_dim), int(bool(interleaved)), _p(positions), _p(slots),
-        _p(q_out), _p(k_cache), _p(v_cache), int(k_cache.shape[2]), T, nq, nkv, d,
+        _p(q_out), _p(k_cache), _p(v_cache), int(k_cache.shape[2]), T, nq, nkv, d, d,
         int(bool(v_grouped)), int(vector_min_tokens), _stream()))
     return q_out
 
@@ -1865,6 +1865,9 @@ def stream_start(resid: torch.Tensor, pending: Optional[torch.Tensor], factor: f
 
 
 # ---- a projection's heads made ready one by one: rotation, then a unit norm ---------------------------------
+HEAD_ROWS_VECTOR = 128        # tokens from which bfloat16 heads without a unit norm are made ready eight dims a lane
+
+
 def head_rows(qkv: torch.Tensor, slots: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, num_heads: int,
               num_kv_heads: int, head_dim: int, value_dim: int, v_grouped: bool = False, cos: Optional[torch.Tensor] = None,
               sin: Optional[torch.Tensor] = None, rotary_dim: int = 0, interleaved: bool = False,
@@ -1901,6 +1904,15 @@ def head_rows(qkv: torch.Tensor, slots: torch.Tensor, k_cache: torch.Tensor, v_c
             if w.shape != (n,):
                 raise KernelError(f"head_rows: a bias or weight of {tuple(w.shape)} is not [{n}]")
     q_out = torch.empty((T, nq, d), dtype=qkv.dtype, device=qkv.device)
+    if (qkv.dtype == torch.bfloat16 and v_grouped and not unit_norm and T >= HEAD_ROWS_VECTOR and d % 8 == 0 and dv % 8 == 0
+            and max(d, dv) <= 256 and (interleaved or rot % 16 == 0) and positions is not None):
+        # many tokens: the vectorized form of `qk_norm_rope_kv`
+        none = _p(None)
+        _ok(lib().xi_qk_norm_rope_kv(
+            _p(qkv), BF16, 0, _p(bias), _p(q_weight), _p(k_weight), ctypes.c_float(eps), _p(cos) if rot else none, _p(sin) if rot else none,
+            rot, int(bool(interleaved)), _p(positions), _p(slots), _p(q_out), _p(k_cache), _p(v_cache),
+            int(k_cache.shape[2]), T, nq, nkv, d, dv, 1, HEAD_ROWS_VECTOR, _stream()))
+        return q_out
     _ok(lib().xi_head_rows(_p(qkv), _code(qkv, "head_rows"), _p(slots), _p(q_out), _p(k_cache), _p(v_cache),
                            int(k_cache.shape[2]), T, nq, nkv, d, dv, int(bool(v_grouped)), _p(cos if rot else None),
                            _p(sin if rot else None), rot, int(bool(interleaved)), _p(positions if rot else None),
