@@ -57,7 +57,8 @@ __device__ __forceinline__ float decay_of(float z, float inv_tau) {
 
 // ONE: a token's decay is one number for all of a head's channels (a constant per head, or from a step size): every
 // thread makes it itself and keeps it in a register, and the decays' row in LDS is neither written nor read.
-template <typename T, int RPT, bool ONE>
+// ACT: q, k and v pass silu.
+template <typename T, int RPT, bool ONE, bool ACT>
 __global__ __launch_bounds__(kScanWaves* kWave) void linear_scan_kernel(
     const T* __restrict__ q, long long q_stride, const T* __restrict__ k, long long k_stride, const T* __restrict__ v,
     long long v_stride, const float* __restrict__ z, const float* __restrict__ z_bias, float inv_tau,
@@ -66,7 +67,7 @@ __global__ __launch_bounds__(kScanWaves* kWave) void linear_scan_kernel(
     int group_heads, const float* __restrict__ state_in, long long in_stride, const long long* __restrict__ in_idx,
     float* __restrict__ state_out, long long out_stride, const long long* __restrict__ out_idx,
     const int* __restrict__ first, const int* __restrict__ last, float* __restrict__ out, float* __restrict__ decay_out,
-    int H, int dk, int dv, float q_scale, float k_scale, int act) {
+    int H, int dk, int dv, float q_scale, float k_scale) {
   __shared__ __attribute__((aligned(16))) float qs[2][kScanWaves * 64], ks[2][kScanWaves * 64], as[2][kScanWaves * 64];
   __shared__ float part[2][kScanWaves][kScanCols];
   __shared__ float npart[2][kScanWaves];
@@ -100,7 +101,7 @@ __global__ __launch_bounds__(kScanWaves* kWave) void linear_scan_kernel(
   };
   auto read = [&](T x) {
     const float f = to_float(x);
-    return act ? f / (1.f + expf(-f)) : f;
+    return ACT ? f / (1.f + expf(-f)) : f;
   };
   auto fetch = [&](int t, float dt, float& fq, float& fk, float& fa) {      // (channels past the head's stay zero)
     if (c < dk) {
@@ -320,7 +321,7 @@ int xi_linear_scan(const void* q, long long q_stride, const void* k, long long k
   XI_CHECK((in_idx == nullptr || (state_in && in_stride >= (long long)H * dk * dv)) &&
                (out_idx == nullptr || (state_out && out_stride >= (long long)H * dk * dv)),
            "linear_scan: states need a place of at least H dk dv floats each");
-  XI_CHECK(act == 0 || act == 1, "linear_scan: unknown activation %d", act);
+  XI_CHECK(act == 0 || (act == 1 && z == nullptr), "linear_scan: activation %d (silu comes with one decay a head and token)", act);
   XI_CHECK(first && last, "linear_scan: the items' token ranges are missing");
   if (n_items == 0) return 0;
   dim3 grid((unsigned)n_items, (unsigned)H, (unsigned)((v_cols + kScanCols - 1) / kScanCols));
@@ -330,11 +331,12 @@ int xi_linear_scan(const void* q, long long q_stride, const void* k, long long k
 #define XI_SCAN_ARGS(TT)                                                                                                      \
       (const TT*)q, q_stride, (const TT*)k, k_stride, (const TT*)v, v_stride, z, z_bias, inv_tau, head_decay, (const TT*)step,    \
       step_stride, step_bias, decay_log, gates, v_cols, group_heads, state_in, in_stride,                                                    \
-      in_idx, state_out, out_stride, out_idx, first, last, out, decay_out, H, dk, dv, q_scale, k_scale, act
+      in_idx, state_out, out_stride, out_idx, first, last, out, decay_out, H, dk, dv, q_scale, k_scale
 #define XI_SCAN(TT, R)                                                                                                        \
   do {                                                                                                                        \
-    if (z) linear_scan_kernel<TT, R, false><<<grid, kScanWaves * kWave, 0, stream>>>(XI_SCAN_ARGS(TT));                       \
-    else linear_scan_kernel<TT, R, true><<<grid, kScanWaves * kWave, 0, stream>>>(XI_SCAN_ARGS(TT));                          \
+    if (z) linear_scan_kernel<TT, R, false, false><<<grid, kScanWaves * kWave, 0, stream>>>(XI_SCAN_ARGS(TT));                \
+    else if (act) linear_scan_kernel<TT, R, true, true><<<grid, kScanWaves * kWave, 0, stream>>>(XI_SCAN_ARGS(TT));           \
+    else linear_scan_kernel<TT, R, true, false><<<grid, kScanWaves * kWave, 0, stream>>>(XI_SCAN_ARGS(TT));                   \
   } while (0)
 #define XI_SCAN_T(TT)            \
   do {                           \

@@ -121,14 +121,14 @@ __device__ __forceinline__ void store8(bf16* p, const float (&v)[8]) {
 // The convolution for a thread's 8 channels over a run of `run` tokens: the last TAPS - 1 inputs stay in registers
 // from token to token, so a row of u is read once; at a run's first token they come from the rows before (or the
 // request's tail), at a sequence's first token from its tail.  The sums are those of `causal_conv_kernel`, term by term.
-template <typename T, int TAPS>
+template <typename T, int TAPS, bool ACT, bool INB>      // ACT: silu on the result; INB: the inputs have a bias
 __global__ __launch_bounds__(256) void causal_conv_run_kernel(const T* __restrict__ u, long long u_stride,
                                                               const float* __restrict__ w, const float* __restrict__ bias,
                                                               const float* __restrict__ tails, long long slot_stride,
                                                               const long long* __restrict__ slots,
                                                               const int* __restrict__ tok_seq, const int* __restrict__ cu_q,
                                                               T* __restrict__ out, int n_tok, int C, int run,
-                                                              const float* __restrict__ in_bias, int act) {
+                                                              const float* __restrict__ in_bias) {
   const int c = 8 * (blockIdx.y * blockDim.x + threadIdx.x);
   if (c >= C) return;
   const int ta = blockIdx.x * run;
@@ -137,7 +137,7 @@ __global__ __launch_bounds__(256) void causal_conv_run_kernel(const T* __restric
 #pragma unroll
   for (int i = 0; i < 8; ++i) {
     bs[i] = bias[c + i];
-    ib[i] = in_bias ? in_bias[c + i] : 0.f;
+    ib[i] = INB ? in_bias[c + i] : 0.f;
 #pragma unroll
     for (int j = 0; j < TAPS; ++j) wt[j][i] = w[(size_t)(c + i) * TAPS + j];
   }
@@ -154,7 +154,8 @@ __global__ __launch_bounds__(256) void causal_conv_run_kernel(const T* __restric
         if (s >= t0) {
           load8(u + (size_t)s * u_stride + c, win[i]);
 #pragma unroll
-          for (int e = 0; e < 8; ++e) win[i][e] += ib[e];
+          for (int e = 0; e < 8; ++e)
+            if constexpr (INB) win[i][e] += ib[e];
         } else {
           load8(tail + (size_t)(TAPS - 1 - (t0 - s)) * C + c, win[i]);      // (kept with their bias)
         }
@@ -164,12 +165,12 @@ __global__ __launch_bounds__(256) void causal_conv_run_kernel(const T* __restric
     load8(u + (size_t)t * u_stride + c, cur);
 #pragma unroll
     for (int i = 0; i < 8; ++i) {
-      cur[i] += ib[i];
+      if constexpr (INB) cur[i] += ib[i];
       float acc = bs[i];
 #pragma unroll
       for (int j = 0; j < TAPS - 1; ++j) acc = fmaf(wt[j][i], win[j][i], acc);
       acc = fmaf(wt[TAPS - 1][i], cur[i], acc);
-      o[i] = act ? acc / (1.f + expf(-acc)) : acc;
+      o[i] = ACT ? acc / (1.f + expf(-acc)) : acc;
     }
     store8(out + (size_t)t * C + c, o);
 #pragma unroll
@@ -266,9 +267,16 @@ int xi_causal_conv(const void* u, long long u_stride, int dtype, const float* w,
       (reinterpret_cast<uintptr_t>(out) & 15) == 0 && esize) {
     const int run = n_tok >= 1024 ? 8 : n_tok >= 256 ? 4 : 1;
     dim3 vgrid((unsigned)((n_tok + run - 1) / run), (unsigned)((C / 8 + 255) / 256));
-#define XI_CONV_RUN(TT, TAPS)                                                                                          \
-  causal_conv_run_kernel<TT, TAPS><<<vgrid, 256, 0, stream>>>((const TT*)u, u_stride, w, bias, tails, slot_stride, slots, \
-                                                             tok_seq, cu_q, (TT*)out, n_tok, C, run, in_bias, act)
+#define XI_CONV_RUN_AB(TT, TAPS, ACT, INB)                                                                                  \
+  causal_conv_run_kernel<TT, TAPS, ACT, INB><<<vgrid, 256, 0, stream>>>((const TT*)u, u_stride, w, bias, tails, slot_stride, \
+                                                                       slots, tok_seq, cu_q, (TT*)out, n_tok, C, run, in_bias)
+#define XI_CONV_RUN(TT, TAPS)                               \
+  do {                                                      \
+    if (act && in_bias) XI_CONV_RUN_AB(TT, TAPS, true, true); \
+    else if (act) XI_CONV_RUN_AB(TT, TAPS, true, false);    \
+    else if (in_bias) XI_CONV_RUN_AB(TT, TAPS, false, true); \
+    else XI_CONV_RUN_AB(TT, TAPS, false, false);            \
+  } while (0)
 #define XI_CONV_TAPS(TT)              \
   switch (taps) {                     \
     case 1: XI_CONV_RUN(TT, 1); break; \
@@ -284,6 +292,7 @@ int xi_causal_conv(const void* u, long long u_stride, int dtype, const float* w,
     }
 #undef XI_CONV_TAPS
 #undef XI_CONV_RUN
+#undef XI_CONV_RUN_AB
     XI_LAUNCH_CHECK("causal_conv");
     return 0;
   }

@@ -367,7 +367,7 @@ def linear_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: torch.
     Or `gates` float32 [T, H, 2], made beforehand: a = gates[t, h, 0] and the token's value row times gates[t, h, 1].
     `value_cols` = value_dim - 1: v is [T, H (value_dim - 1)] and the state's last column reads the value 1 (it then
     holds the decayed sum of the weighted keys alone, and the results' last column that sum times q).
-    `silu`: q, k and v pass silu first (in float32, before any factor).
+    `silu` (not beside `z`): q, k and v pass silu first (in float32, before any factor).
     `groups` G: q and k are [T, G dk] and head h reads the columns of group h // (H / G).
     state float32 [slots, H, dk, dv] (slots may be strided); state_slots int64 [B]; cu_q int32 [B + 1].
     Returns o float32 [T, H, dv].
@@ -379,6 +379,8 @@ def linear_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state: torch.
     the index arrays of this cutting are kept for the next layer."""
     H, dk, dv = int(heads), int(key_dim), int(value_dim)
     T = q.shape[0]
+    if silu and z is not None:
+        raise KernelError("linear_scan: silu on q, k and v comes with one decay a head and token")
     G = H if groups is None else int(groups)
     if G <= 0 or H % G:
         raise KernelError(f"linear_scan: {H} heads in {G} groups")
