@@ -307,6 +307,9 @@ __global__ void qk_norm_rope_kv_kernel(const void* __restrict__ qkv_v, int slice
 // workgroup of a V head turns its [tokens, d] tile through LDS so that a wave's store takes eight
 // tokens by eight dims: where the eight tokens follow each other in a group of the pool, one line
 // of 128 bytes.  Value heads may have a size of their own, dv.
+// Rows may be longer than their heads (`width`), the values' first column is `v_col` (behind the keys, or the keys' own: the
+// values are then the keys as projected), and with `vcos` / `vsin` (float32 [positions, dv / 2]; dv % 16 == 0) value heads turn
+// by their position in pairs (i, i + dv / 2).
 // Needs d % 8 == 0, dv % 8 == 0 and, for the half layout, rotary_dim % 16 == 0 (the partner of a lane's
 // 8 elements is then another lane's 8 elements).
 struct alignas(16) bf16x8v { bf16 v[8]; };
@@ -315,10 +318,10 @@ __global__ __launch_bounds__(1024) void qk_norm_rope_kvt_bf16_kernel(
     const bf16* __restrict__ qkv, const float* __restrict__ bias, const float* __restrict__ qw, const float* __restrict__ kw, float eps,
     const float* __restrict__ cos_t, const float* __restrict__ sin_t, int rot, int interleaved,
     const int* __restrict__ positions, const long long* __restrict__ slots, bf16* __restrict__ q_out,
-    bf16* __restrict__ k_cache, bf16* __restrict__ vt_cache, int page_size, int n_tok, int nq, int nkv, int d, int dv) {
+    bf16* __restrict__ k_cache, bf16* __restrict__ vt_cache, int page_size, int n_tok, int nq, int nkv, int d, int dv,
+    long long width, int v_col, const float* __restrict__ vcos, const float* __restrict__ vsin) {
   extern __shared__ __align__(16) unsigned char smem_raw[];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
-  const size_t width = (size_t)(nq + nkv) * d + (size_t)nkv * dv;      // of a packed row
   const int lph = d >> 3;          // lanes per head
   const int hpw = 64 / lph;        // tokens a wave holds
   const int tpw = (blockDim.x >> 6) * hpw;   // tokens of the workgroup (at most 64)
@@ -344,7 +347,8 @@ __global__ __launch_bounds__(1024) void qk_norm_rope_kvt_bf16_kernel(
       const int off = (int)(slot - page * page_size);
       place = ((unsigned long long)page * nkv + kvh) * dv * page_size + (unsigned long long)(off >> 3) * dv * 8 + (off & 7);
     }
-    const size_t col0 = (size_t)(nq + nkv) * d + (size_t)kvh * dv;
+    const size_t col0 = (size_t)v_col + (size_t)kvh * dv;
+    const int vhalf = dv >> 1;
     for (int u = tid; u < tpw * (dv >> 3); u += (int)blockDim.x) {
       const int tok = u / (dv >> 3), cc = 8 * (u - tok * (dv >> 3));
       if (t0 + tok >= n_tok) break;
@@ -353,6 +357,27 @@ __global__ __launch_bounds__(1024) void qk_norm_rope_kvt_bf16_kernel(
         bf16x8v x = *reinterpret_cast<const bf16x8v*>(&raw);
 #pragma unroll
         for (int e = 0; e < 8; ++e) x.v[e] = from_float<bf16>(to_float(x.v[e]) + bias[col0 + cc + e]);
+        raw = *reinterpret_cast<const uint4*>(&x);
+      }
+      if (vcos) {                      // this chunk turned with its partner half a head away
+        const bool first = cc < vhalf;
+        const int pc = first ? cc + vhalf : cc - vhalf, p0 = first ? cc : pc;
+        bf16x8v x = *reinterpret_cast<const bf16x8v*>(&raw);
+        bf16x8v y = *reinterpret_cast<const bf16x8v*>(qkv + (size_t)(t0 + tok) * width + col0 + pc);
+        if (bias) {
+#pragma unroll
+          for (int e = 0; e < 8; ++e) y.v[e] = from_float<bf16>(to_float(y.v[e]) + bias[col0 + pc + e]);
+        }
+        const size_t at = (size_t)positions[t0 + tok] * vhalf + p0;
+        const float4 c0 = *reinterpret_cast<const float4*>(vcos + at), c1 = *reinterpret_cast<const float4*>(vcos + at + 4);
+        const float4 s0 = *reinterpret_cast<const float4*>(vsin + at), s1 = *reinterpret_cast<const float4*>(vsin + at + 4);
+        const float cs[8] = {c0.x, c0.y, c0.z, c0.w, c1.x, c1.y, c1.z, c1.w};
+        const float sn[8] = {s0.x, s0.y, s0.z, s0.w, s1.x, s1.y, s1.z, s1.w};
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+          const float xv = to_float(x.v[e]), yv = to_float(y.v[e]);
+          x.v[e] = from_float<bf16>(first ? xv * cs[e] - yv * sn[e] : xv * cs[e] + yv * sn[e]);
+        }
         raw = *reinterpret_cast<const uint4*>(&x);
       }
       unsigned* dst = reinterpret_cast<unsigned*>(vs + tok * vstride + cc);
@@ -1029,12 +1054,21 @@ int xi_silu_mul(const void* gate_up, void* out, int dtype, int n_tok, int I, hip
 
 // qkv: [T, heads * d] in `dtype`, or, with slices > 0, float32 partial sums [slices, T, heads * d]
 // of it (then `dtype` is that of q_out and the cache, and the form of one wave per head runs).  dv: the value heads' size;
-// one that is not d is for the vectorized form alone (bfloat16, V in groups of eight keys, sizes in eights).
+// one that is not d is for the vectorized form alone (bfloat16, V in groups of eight keys, sizes in eights), and so are
+// row_stride (elements from row to row; 0: the heads side by side), v_col (the values' first column; -1: behind the keys) and
+// vcos / vsin (float32 [positions, dv / 2], value heads turned in pairs (i, i + dv / 2); null: not).
 int xi_qk_norm_rope_kv(const void* qkv, int dtype, int slices, const float* bias, const float* qw, const float* kw, float eps,
                        const float* cos_t, const float* sin_t, int rot, int interleaved,
                        const int* positions, const long long* slots, void* q_out, void* k_cache,
                        void* v_cache, int page_size, int n_tok, int nq, int nkv, int d, int dv, int v_grouped,
-                       int vector_min_tokens, hipStream_t stream) {
+                       int vector_min_tokens, long long row_stride, int v_col, const float* vcos, const float* vsin,
+                       hipStream_t stream) {
+  const long long heads_width = (long long)(nq + nkv) * d + (long long)nkv * dv;
+  if (row_stride == 0) row_stride = heads_width;
+  if (v_col < 0) v_col = (nq + nkv) * d;
+  XI_CHECK(row_stride >= (long long)v_col + (long long)nkv * dv && row_stride >= (long long)(nq + nkv) * d,
+           "qk_norm_rope_kv: rows of %lld do not hold the heads", row_stride);
+  XI_CHECK((vcos == nullptr) == (vsin == nullptr), "qk_norm_rope_kv: the values' tables come together");
   XI_CHECK(n_tok >= 0 && nq > 0 && nkv > 0 && d > 0 && page_size > 0,
            "qk_norm_rope_kv: bad sizes T=%d nq=%d nkv=%d d=%d page=%d", n_tok, nq, nkv, d, page_size);
   XI_CHECK(rot >= 0 && rot <= d && rot % 2 == 0, "qk_norm_rope_kv: rotary_dim %d must be even and <= head_dim %d", rot, d);
@@ -1048,7 +1082,8 @@ int xi_qk_norm_rope_kv(const void* qkv, int dtype, int slices, const float* bias
            page_size);
   if (slices == 0 && n_tok >= vector_min_tokens && dtype == kBF16 && v_grouped && d % 8 == 0 && d <= 256 &&
       dv % 8 == 0 && dv > 0 && dv <= 256 &&
-      (interleaved || rot % 16 == 0) &&
+      (interleaved || rot % 16 == 0) && row_stride % 8 == 0 && v_col % 8 == 0 &&
+      (vcos == nullptr || (!interleaved && dv % 16 == 0 && ((uintptr_t)vcos | (uintptr_t)vsin) % 16 == 0)) &&
       ((uintptr_t)qkv | (uintptr_t)q_out | (uintptr_t)k_cache | (uintptr_t)cos_t | (uintptr_t)sin_t) % 16 == 0) {
     const int lph = d / 8, hpw = 64 / lph;
     int n_waves = 64 / hpw;                       // waves of a workgroup: at most 64 tokens, at most 16 waves
@@ -1059,10 +1094,12 @@ int xi_qk_norm_rope_kv(const void* qkv, int dtype, int slices, const float* bias
     const size_t lds = (size_t)tpw * (dv + 2) * sizeof(bf16);
     qk_norm_rope_kvt_bf16_kernel<<<dim3(blocks_x, nq + 2 * nkv), n_waves * 64, lds, stream>>>(
         (const bf16*)qkv, bias, qw, kw, eps, cos_t, sin_t, rot, interleaved, positions, slots, (bf16*)q_out,
-        (bf16*)k_cache, (bf16*)v_cache, page_size, n_tok, nq, nkv, d, dv);
+        (bf16*)k_cache, (bf16*)v_cache, page_size, n_tok, nq, nkv, d, dv, row_stride, v_col, vcos, vsin);
     XI_LAUNCH_CHECK("qk_norm_rope_kv");
     return 0;
   }
+  XI_CHECK(row_stride == heads_width && v_col == (nq + nkv) * d && vcos == nullptr,
+           "qk_norm_rope_kv: longer rows, values in the keys' columns or turned values need the vectorized form");
   XI_CHECK(dv == d, "qk_norm_rope_kv: value heads of %d beside keys of %d need the vectorized form", dv, d);
   const long long waves = (long long)n_tok * (nq + 2 * nkv);
   const int wpb = 4;

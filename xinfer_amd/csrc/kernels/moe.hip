@@ -10,7 +10,12 @@
 //   expert   y_e = Wd_e (act(Wg_e x) * (Wu_e x)), no biases; gate and up of all experts are stacked
 //            [E, 2F, H] (gate rows first), down [E, H, F]; or without a gate, y_e = Wd_e act(Wu_e x)
 //            with the up rows alone, [E, F, H].
-//   output   sum over the chosen experts, in the order they were chosen, of weight * y_e: float32.
+//   output   sum over the chosen experts, in the order they were chosen, of weight * y_e, then (if given) a further
+//            row of the token (a shared branch's result): float32.
+//            With a correction c [E] (scores over all experts or sigmoids) the experts are chosen by s + c
+//            and weighted by s without it.
+//   identity The last I of the router's outputs may stand for experts without tensors whose output is x
+//            itself: a pair whose expert is E or above adds weight * x.
 //   `scores` 2: the weights are sigmoid(z) of the chosen experts, as they are (the largest z are the largest scores).
 //   A weight may instead multiply the expert's INPUT, y_e = expert(weight * x) (`in_wt` of the gate/up product: the
 //   products are linear, so the weight multiplies their float32 sums before the activation; the down product then
@@ -35,8 +40,10 @@ __global__ __launch_bounds__(kRouteWaves* kWave) void moe_route_kernel(const T* 
                                                                        const float* __restrict__ wr,
                                                                        const float* __restrict__ br, int* __restrict__ idx,
                                                                        float* __restrict__ wt, int H, int E, int top,
-                                                                       int all_scores, float* __restrict__ extra, int X) {
+                                                                       int all_scores, float* __restrict__ extra, int X,
+                                                                       const float* __restrict__ correction) {
   __shared__ float z[kMaxExperts];
+  __shared__ float score[kMaxExperts];       // with a correction: the scores the weights are made of
   __shared__ float denom_all[2];
   __shared__ float chosen[kMaxTop];
   const int t = blockIdx.x;
@@ -79,6 +86,15 @@ __global__ __launch_bounds__(kRouteWaves* kWave) void moe_route_kernel(const T* 
     __builtin_amdgcn_s_waitcnt(0);
     __builtin_amdgcn_wave_barrier();
   }
+  if (correction) {          // chosen by the corrected scores (a lane reads back what it wrote itself)
+    for (int e = lane; e < E; e += kWave) {
+      const float s = all_scores == 2 ? 1.f / (1.f + expf(-z[e])) : expf(z[e] - denom_all[0]) / denom_all[1];
+      score[e] = s;
+      z[e] = s + correction[e];
+    }
+    __builtin_amdgcn_s_waitcnt(0);
+    __builtin_amdgcn_wave_barrier();
+  }
   for (int r = 0; r < top; ++r) {
     float best = -INFINITY;
     int at = 0x7fffffff;
@@ -99,13 +115,17 @@ __global__ __launch_bounds__(kRouteWaves* kWave) void moe_route_kernel(const T* 
     if (at >= E) at = E - 1;            // no finite logit left (rows of NaN): any valid expert
     if (lane == 0) {
       idx[(size_t)t * top + r] = at;
-      chosen[r] = best;
+      chosen[r] = correction ? score[at] : best;
       z[at] = -INFINITY;
     }
     __builtin_amdgcn_s_waitcnt(0);      // lane 0's write to LDS is done before the wave reads z again
     __builtin_amdgcn_wave_barrier();
   }
-  if (lane == 0 && all_scores == 2) {
+  if (lane == 0 && correction) {
+    float sum = 0.f;
+    for (int r = 0; r < top; ++r) sum += chosen[r];
+    for (int r = 0; r < top; ++r) wt[(size_t)t * top + r] = all_scores == 2 ? chosen[r] : chosen[r] / (sum + 1e-20f);
+  } else if (lane == 0 && all_scores == 2) {
     for (int r = 0; r < top; ++r) wt[(size_t)t * top + r] = 1.f / (1.f + expf(-chosen[r]));
   } else if (lane == 0 && all_scores) {
     const float m = denom_all[0], d = denom_all[1];
@@ -133,11 +153,12 @@ constexpr int kMoeWaves = 4;
 template <typename T, int ACT, bool GATED>
 __global__ __launch_bounds__(kMoeWaves* kWave) void moe_gate_up_kernel(const T* __restrict__ x, const T* __restrict__ wgu,
                                                                        const int* __restrict__ idx, T* __restrict__ mid,
-                                                                       int H, int F, int top, int FT,
+                                                                       int H, int F, int E, int top, int FT,
                                                                        const float* __restrict__ in_wt) {
   extern __shared__ float xs[];
   const int pair = blockIdx.x, t = pair / top;
   const int e = idx[pair];
+  if (e >= E) return;                 // an identity expert: nothing to multiply
   const float wi = in_wt ? in_wt[pair] : 1.f;
   const int lane = threadIdx.x & (kWave - 1), wave = threadIdx.x / kWave;
   for (int k = threadIdx.x; k < H; k += blockDim.x) xs[k] = to_float(x[(size_t)t * H + k]);
@@ -182,7 +203,9 @@ __global__ __launch_bounds__(kMoeWaves* kWave) void moe_gate_up_kernel(const T* 
 template <typename T>
 __global__ __launch_bounds__(kMoeWaves* kWave) void moe_down_kernel(const T* __restrict__ mid, const T* __restrict__ wd,
                                                                     const int* __restrict__ idx, const float* __restrict__ wt,
-                                                                    float* __restrict__ out, int H, int F, int top, int NTile) {
+                                                                    float* __restrict__ out, int H, int F, int E, int top,
+                                                                    int NTile, const T* __restrict__ x,
+                                                                    const T* __restrict__ add) {
   extern __shared__ float ms[];       // [top, F]
   const int t = blockIdx.x;
   const int lane = threadIdx.x & (kWave - 1), wave = threadIdx.x / kWave;
@@ -192,7 +215,12 @@ __global__ __launch_bounds__(kMoeWaves* kWave) void moe_down_kernel(const T* __r
   for (int n = blockIdx.y * NTile + wave; n < n_end; n += kMoeWaves) {
     float total = 0.f;
     for (int r = 0; r < top; ++r) {
-      const T* w = wd + ((size_t)idx[(size_t)t * top + r] * H + n) * F;
+      const int e = idx[(size_t)t * top + r];
+      if (e >= E) {                   // an identity expert: the input itself
+        total += wt[(size_t)t * top + r] * to_float(x[(size_t)t * H + n]);
+        continue;
+      }
+      const T* w = wd + ((size_t)e * H + n) * F;
       float acc = 0.f;
       if (sizeof(T) == 2 && F % 8 == 0) {
         for (int f = 8 * lane; f < F; f += 8 * kWave) {
@@ -206,7 +234,7 @@ __global__ __launch_bounds__(kMoeWaves* kWave) void moe_down_kernel(const T* __r
       acc = wave_sum(acc);
       total += wt[(size_t)t * top + r] * acc;
     }
-    if (lane == 0) out[(size_t)t * H + n] = total;
+    if (lane == 0) out[(size_t)t * H + n] = add ? total + to_float(add[(size_t)t * H + n]) : total;
   }
 }
 
@@ -218,8 +246,10 @@ extern "C" {
 
 // x [T, H] in `dtype`; wr float32 [E, H]; br float32 [E] or null; idx int32 [T, top]; wt float32 [T, top].
 // all_scores: 0, 1 (see the head of the file) or 2 (sigmoid of the chosen logits).  extra float32 [T, X]: the products with rows E .. E + X - 1 of wr (X may be 0).
+// correction float32 [E] or null (with all_scores 1 or 2): added to the scores for the choice alone.
 int xi_moe_route(const void* x, int dtype, const float* wr, const float* br, int* idx, float* wt, int n_tok, int H, int E,
-                 int top, int all_scores, float* extra, int X, hipStream_t stream) {
+                 int top, int all_scores, float* extra, int X, const float* correction, hipStream_t stream) {
+  XI_CHECK(correction == nullptr || all_scores != 0, "moe_route: a correction is added to scores over all experts");
   XI_CHECK(X >= 0 && (X == 0 || extra != nullptr), "moe_route: %d further rows need a place for their results", X);
   XI_CHECK(n_tok >= 0 && H > 0 && E > 0 && E <= kMaxExperts, "moe_route: bad sizes T=%d H=%d experts=%d (at most %d)", n_tok,
            H, E, kMaxExperts);
@@ -228,10 +258,10 @@ int xi_moe_route(const void* x, int dtype, const float* wr, const float* br, int
   if (n_tok == 0) return 0;
   if (dtype == kF32)
     moe_route_kernel<float><<<n_tok, kRouteWaves * kWave, 0, stream>>>((const float*)x, wr, br, idx, wt, H, E, top, all_scores,
-                                                                       extra, X);
+                                                                       extra, X, correction);
   else if (dtype == kBF16)
     moe_route_kernel<bf16><<<n_tok, kRouteWaves * kWave, 0, stream>>>((const bf16*)x, wr, br, idx, wt, H, E, top, all_scores,
-                                                                      extra, X);
+                                                                      extra, X, correction);
   else
     XI_CHECK(false, "moe_route: unknown dtype %d", dtype);
   XI_LAUNCH_CHECK("moe_route");
@@ -240,7 +270,8 @@ int xi_moe_route(const void* x, int dtype, const float* wr, const float* br, int
 
 // x [T, H], wgu [E, 2F, H], idx [T * top] -> mid [T * top, F] = act(gate) * up, all in `dtype`;
 // gated 0: wgu [E, F, H] and mid = act(up).  act: 0 silu, 1 gelu (tanh form), 2 the square of relu.
-// in_wt float32 [T * top] or null: a weight a pair on the expert's input.
+// in_wt float32 [T * top] or null: a weight a pair on the expert's input.  A pair whose expert is E or above (an identity
+// expert) leaves its row of mid unwritten.
 int xi_moe_gate_up(const void* x, const void* wgu, const int* idx, void* mid, int dtype, int act, int gated, int n_tok, int H,
                    int F, int E, int top, const float* in_wt, hipStream_t stream) {
   XI_CHECK(n_tok >= 0 && H > 0 && F > 0 && E > 0 && top > 0, "moe_gate_up: bad sizes T=%d H=%d F=%d E=%d top=%d", n_tok, H, F, E,
@@ -261,7 +292,7 @@ int xi_moe_gate_up(const void* x, const void* wgu, const int* idx, void* mid, in
       hipError_t e_ = hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds); \
       XI_CHECK(e_ == hipSuccess, "moe_gate_up: cannot get %zu bytes of LDS", lds);                              \
     }                                                                                                           \
-    kern<<<grid, kMoeWaves * kWave, lds, stream>>>((const TT*)x, (const TT*)wgu, idx, (TT*)mid, H, F, top, FT, in_wt); \
+    kern<<<grid, kMoeWaves * kWave, lds, stream>>>((const TT*)x, (const TT*)wgu, idx, (TT*)mid, H, F, E, top, FT, in_wt); \
   } while (0)
 #define XI_GU_A(TT, G)            \
   do {                            \
@@ -280,9 +311,10 @@ int xi_moe_gate_up(const void* x, const void* wgu, const int* idx, void* mid, in
   return 0;
 }
 
-// mid [T * top, F], wd [E, H, F] in `dtype`; idx, wt [T, top] -> out float32 [T, H].
+// mid [T * top, F], wd [E, H, F] in `dtype`; idx, wt [T, top] -> out float32 [T, H].  x [T, H] in `dtype`: what experts
+// numbered E and above return (null: there are none); add [T, H] in `dtype` or null: added to the sum.
 int xi_moe_down(const void* mid, const void* wd, const int* idx, const float* wt, float* out, int dtype, int n_tok, int H,
-                int F, int E, int top, hipStream_t stream) {
+                int F, int E, int top, const void* x, const void* add, hipStream_t stream) {
   XI_CHECK(n_tok >= 0 && H > 0 && F > 0 && E > 0 && top > 0, "moe_down: bad sizes T=%d H=%d F=%d E=%d top=%d", n_tok, H, F, E, top);
   const size_t lds = (size_t)top * F * sizeof(float);
   XI_CHECK(lds <= 64 * 1024, "moe_down: %d rows of %d do not fit in LDS", top, F);
@@ -297,7 +329,8 @@ int xi_moe_down(const void* mid, const void* wd, const int* idx, const float* wt
       hipError_t e_ = hipFuncSetAttribute((const void*)kern, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds); \
       XI_CHECK(e_ == hipSuccess, "moe_down: cannot get %zu bytes of LDS", lds);                                 \
     }                                                                                                           \
-    kern<<<grid, kMoeWaves * kWave, lds, stream>>>((const TT*)mid, (const TT*)wd, idx, wt, out, H, F, top, NTile); \
+    kern<<<grid, kMoeWaves * kWave, lds, stream>>>((const TT*)mid, (const TT*)wd, idx, wt, out, H, F, E, top, NTile, \
+                                                   (const TT*)x, (const TT*)add); \
   } while (0)
   if (dtype == kF32) XI_DN(float);
   else if (dtype == kBF16) XI_DN(bf16);

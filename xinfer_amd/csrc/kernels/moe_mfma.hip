@@ -12,7 +12,9 @@
 //                 hidden rows, kept in slot order); activated form: W the up rows alone, result
 //                 act(up) in bfloat16 (experts without a gate); plain form: float32.
 //   moe_combine   out[t] = sum over the token's chosen experts, in the order they were chosen, of
-//                 weight * row: a fixed order, float32.
+//                 weight * row (an identity expert's row is x[t]), then a further row if given: a fixed
+//                 order, float32.
+// Experts numbered E .. E + I - 1 are identity experts: they get slots behind the others' and no tiles.
 // A row's result depends on its own operands alone (the matrix cores keep rows apart), so it does not
 // matter which other rows share its tile.
 #include "common.h"
@@ -25,24 +27,25 @@ typedef __attribute__((ext_vector_type(4))) float mf32x4;
 constexpr int kSortThreads = 1024;
 constexpr int kSortExperts = 1024;
 
-__global__ __launch_bounds__(kSortThreads) void moe_sort_kernel(const int* __restrict__ idx, int P, int E, int BM,
+__global__ __launch_bounds__(kSortThreads) void moe_sort_kernel(const int* __restrict__ idx, int P, int E, int I, int BM,
                                                                 int* __restrict__ order, int* __restrict__ slot_of,
                                                                 int* __restrict__ tile_expert, int* __restrict__ tile_row0,
                                                                 int* __restrict__ tile_rows, int* __restrict__ n_tiles) {
   __shared__ int count[kSortExperts], cursor[kSortExperts];
-  for (int e = threadIdx.x; e < E; e += kSortThreads) count[e] = 0;
+  const int A = E + I;
+  for (int e = threadIdx.x; e < A; e += kSortThreads) count[e] = 0;
   __syncthreads();
   for (int p = threadIdx.x; p < P; p += kSortThreads) {
     int e = idx[p];
-    e = e < 0 ? 0 : (e >= E ? E - 1 : e);
+    e = e < 0 ? 0 : (e >= A ? A - 1 : e);
     atomicAdd(&count[e], 1);
   }
   __syncthreads();
   if (threadIdx.x == 0) {
     int at = 0, tiles = 0;
-    for (int e = 0; e < E; ++e) {
+    for (int e = 0; e < A; ++e) {
       cursor[e] = at;
-      for (int r = 0; r < count[e]; r += BM) {
+      for (int r = 0; e < E && r < count[e]; r += BM) {
         tile_expert[tiles] = e;
         tile_row0[tiles] = at + r;
         tile_rows[tiles] = count[e] - r < BM ? count[e] - r : BM;
@@ -55,7 +58,7 @@ __global__ __launch_bounds__(kSortThreads) void moe_sort_kernel(const int* __res
   __syncthreads();
   for (int p = threadIdx.x; p < P; p += kSortThreads) {
     int e = idx[p];
-    e = e < 0 ? 0 : (e >= E ? E - 1 : e);
+    e = e < 0 ? 0 : (e >= A ? A - 1 : e);
     const int slot = atomicAdd(&cursor[e], 1);
     order[slot] = p;
     slot_of[p] = slot;
@@ -261,13 +264,66 @@ __global__ __launch_bounds__(256) void moe_group_lds_kernel(const bf16* __restri
 }
 
 __global__ void moe_combine_kernel(const float* __restrict__ y, const int* __restrict__ slot_of, const float* __restrict__ wt,
-                                   float* __restrict__ out, int H, int top) {
+                                   float* __restrict__ out, int H, int top, const int* __restrict__ idx, int E,
+                                   const bf16* __restrict__ x, const bf16* __restrict__ add) {
   const int t = blockIdx.x;
   for (int n = threadIdx.x; n < H; n += blockDim.x) {
     float total = 0.f;
-    for (int r = 0; r < top; ++r) total += wt[(size_t)t * top + r] * y[(size_t)slot_of[(size_t)t * top + r] * H + n];
+    for (int r = 0; r < top; ++r) {
+      const size_t p = (size_t)t * top + r;
+      const bool same = x != nullptr && idx[p] >= E;
+      total += wt[p] * (same ? to_float(x[(size_t)t * H + n]) : y[(size_t)slot_of[p] * H + n]);
+    }
+    if (add) total += to_float(add[(size_t)t * H + n]);
     out[(size_t)t * H + n] = total;
   }
+}
+
+// Rows in whole chunks of four: a thread takes four columns of a row, its pairs' rows asked for four at a time.
+__global__ __launch_bounds__(256) void moe_combine_vec_kernel(const float* __restrict__ y, const int* __restrict__ slot_of,
+                                                              const float* __restrict__ wt, float* __restrict__ out, int H, int top,
+                                                              const int* __restrict__ idx, int E, const bf16* __restrict__ x,
+                                                              const bf16* __restrict__ add) {
+  const int t = blockIdx.x;
+  const int n = 4 * (blockIdx.y * 256 + threadIdx.x);
+  if (n >= H) return;
+  auto four = [](const bf16* p, float (&v)[4]) {
+    const uint2 u = *reinterpret_cast<const uint2*>(p);
+    v[0] = __uint_as_float(u.x << 16);
+    v[1] = __uint_as_float(u.x & 0xffff0000u);
+    v[2] = __uint_as_float(u.y << 16);
+    v[3] = __uint_as_float(u.y & 0xffff0000u);
+  };
+  float total[4] = {0.f, 0.f, 0.f, 0.f}, own[4] = {0.f, 0.f, 0.f, 0.f}, more[4] = {0.f, 0.f, 0.f, 0.f};
+  if (x) four(x + (size_t)t * H + n, own);
+  if (add) four(add + (size_t)t * H + n, more);
+  for (int r0 = 0; r0 < top; r0 += 4) {
+    float4 row[4];
+    float w[4];
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      row[r] = make_float4(0.f, 0.f, 0.f, 0.f);
+      w[r] = 0.f;
+      if (r0 + r >= top) continue;
+      const size_t p = (size_t)t * top + r0 + r;
+      w[r] = wt[p];
+      row[r] = x != nullptr && idx[p] >= E ? make_float4(own[0], own[1], own[2], own[3])
+                                           : *reinterpret_cast<const float4*>(y + (size_t)slot_of[p] * H + n);
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      if (r0 + r >= top) break;
+      total[0] += w[r] * row[r].x;
+      total[1] += w[r] * row[r].y;
+      total[2] += w[r] * row[r].z;
+      total[3] += w[r] * row[r].w;
+    }
+  }
+  if (add) {
+#pragma unroll
+    for (int e = 0; e < 4; ++e) total[e] += more[e];
+  }
+  *reinterpret_cast<float4*>(out + (size_t)t * H + n) = make_float4(total[0], total[1], total[2], total[3]);
 }
 
 }  // namespace xi
@@ -279,11 +335,11 @@ extern "C" {
 // Most tiles of up to `bm` rows that P pairs on E experts can make.
 int xi_moe_tiles_most(int P, int E, int bm) { return (P + bm - 1) / bm + E; }
 
-// idx int32 [P] (expert of every pair) -> order, slot_of int32 [P]; tile_* int32 [xi_moe_tiles_most]; n_tiles int32 [1].
-int xi_moe_sort(const int* idx, int P, int E, int bm, int* order, int* slot_of, int* tile_expert, int* tile_row0,
+// idx int32 [P] (expert of every pair; E .. E + I - 1: identity experts) -> order, slot_of int32 [P]; tile_* int32 [xi_moe_tiles_most]; n_tiles int32 [1].
+int xi_moe_sort(const int* idx, int P, int E, int I, int bm, int* order, int* slot_of, int* tile_expert, int* tile_row0,
                 int* tile_rows, int* n_tiles, hipStream_t stream) {
-  XI_CHECK(P > 0 && E > 0 && E <= kSortExperts && (bm == 32 || bm == 64 || bm == 128), "moe_sort: bad sizes pairs=%d experts=%d rows=%d", P, E, bm);
-  moe_sort_kernel<<<1, kSortThreads, 0, stream>>>(idx, P, E, bm, order, slot_of, tile_expert, tile_row0, tile_rows, n_tiles);
+  XI_CHECK(P > 0 && E > 0 && I >= 0 && E + I <= kSortExperts && (bm == 32 || bm == 64 || bm == 128), "moe_sort: bad sizes pairs=%d experts=%d rows=%d", P, E, bm);
+  moe_sort_kernel<<<1, kSortThreads, 0, stream>>>(idx, P, E, I, bm, order, slot_of, tile_expert, tile_row0, tile_rows, n_tiles);
   XI_LAUNCH_CHECK("moe_sort");
   return 0;
 }
@@ -331,11 +387,18 @@ int xi_moe_group(const void* A, const int* order, int top, const void* W, const 
   return 0;
 }
 
-// y float32 [P, H] in slot order -> out float32 [T, H]
-int xi_moe_combine(const float* y, const int* slot_of, const float* wt, float* out, int n_tok, int H, int top,
-                   hipStream_t stream) {
+// y float32 [P, H] in slot order -> out float32 [T, H].  x bfloat16 [T, H] with idx int32 [T, top]: what experts numbered E and
+// above return (null: there are none); add bfloat16 [T, H] or null: added to the sum.
+int xi_moe_combine(const float* y, const int* slot_of, const float* wt, float* out, int n_tok, int H, int top, const int* idx, int E,
+                   const void* x, const void* add, hipStream_t stream) {
   XI_CHECK(n_tok > 0 && H > 0 && top > 0, "moe_combine: bad sizes T=%d H=%d top=%d", n_tok, H, top);
-  moe_combine_kernel<<<n_tok, 256, 0, stream>>>(y, slot_of, wt, out, H, top);
+  XI_CHECK(x == nullptr || idx != nullptr, "moe_combine: identity experts need the choice");
+  auto whole = [](const void* p, uintptr_t bytes) { return reinterpret_cast<uintptr_t>(p) % bytes == 0; };
+  if (H % 4 == 0 && whole(y, 16) && whole(out, 16) && whole(x, 8) && whole(add, 8))
+    moe_combine_vec_kernel<<<dim3((unsigned)n_tok, (unsigned)((H / 4 + 255) / 256)), 256, 0, stream>>>(
+        y, slot_of, wt, out, H, top, idx, E, (const bf16*)x, (const bf16*)add);
+  else
+    moe_combine_kernel<<<n_tok, 256, 0, stream>>>(y, slot_of, wt, out, H, top, idx, E, (const bf16*)x, (const bf16*)add);
   XI_LAUNCH_CHECK("moe_combine");
   return 0;
 }

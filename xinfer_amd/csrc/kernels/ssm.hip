@@ -8,6 +8,8 @@
 // is cleared when its request starts).  Sums in float32, one rounding.
 // `conv_tail_kernel` then moves the tail on by the step's tokens (a launch of its own: the tail is read by the
 // portion's first tokens and written from its last, which other workgroups hold).
+// `conv_step_kernel`: a step in which every sequence brings one token; the thread that makes a channel's result moves
+// its tail on as well.  The sums are those of `causal_conv_kernel`, term by term.
 //
 // `gated_group_norm_kernel`: v = (y + D[h] x) * silu(z); each of `groups` equal parts of a token's row divided by
 // its own root mean square (eps inside the root), times a weight as long as the row; y float32 [T, heads, dv] (the
@@ -60,6 +62,28 @@ __global__ __launch_bounds__(256) void conv_tail_kernel(const T* __restrict__ u,
     const int s = t1 - (taps - 1) + i;
     tail[(size_t)i * C + c] = s >= t0 ? to_float(u[(size_t)s * u_stride + c]) + ib : tail[(size_t)(i + n) * C + c];
   }
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void conv_step_kernel(const T* __restrict__ u, long long u_stride, const float* __restrict__ w,
+                                                        const float* __restrict__ bias, float* __restrict__ tails,
+                                                        long long slot_stride, const long long* __restrict__ slots,
+                                                        T* __restrict__ out, int C, int taps, const float* __restrict__ in_bias,
+                                                        int act) {
+  const int b = blockIdx.x;
+  const int c = blockIdx.y * blockDim.x + threadIdx.x;
+  if (c >= C) return;
+  float* tail = tails + (size_t)slots[b] * slot_stride + c;
+  const float cur = to_float(u[(size_t)b * u_stride + c]) + (in_bias ? in_bias[c] : 0.f);
+  float acc = bias[c];
+  for (int j = 0; j < taps - 1; ++j) {
+    const float x = tail[(size_t)j * C];
+    acc = fmaf(w[(size_t)c * taps + j], x, acc);
+    if (j > 0) tail[(size_t)(j - 1) * C] = x;
+  }
+  if (taps > 1) tail[(size_t)(taps - 2) * C] = cur;
+  acc = fmaf(w[(size_t)c * taps + taps - 1], cur, acc);
+  out[(size_t)b * C + c] = from_float<T>(act ? acc / (1.f + expf(-acc)) : acc);
 }
 
 template <typename T>
@@ -182,6 +206,46 @@ __global__ __launch_bounds__(256) void causal_conv_run_kernel(const T* __restric
       for (int i = 0; i < 8; ++i) win[TAPS > 1 ? TAPS - 2 : 0][i] = cur[i];
     }
   }
+}
+
+// A step of single tokens, four channels a thread (a step of few requests has no more threads than it needs in flight).
+template <typename T, int TAPS, bool ACT, bool INB>
+__global__ __launch_bounds__(64) void conv_step_vec_kernel(const T* __restrict__ u, long long u_stride, const float* __restrict__ w,
+                                                           const float* __restrict__ bias, float* __restrict__ tails,
+                                                           long long slot_stride, const long long* __restrict__ slots,
+                                                           T* __restrict__ out, int C, const float* __restrict__ in_bias) {
+  const int b = blockIdx.x;
+  const int c = 4 * (blockIdx.y * blockDim.x + threadIdx.x);
+  if (c >= C) return;
+  float wt[4 * TAPS], win[TAPS][4], acc[4];
+#pragma unroll
+  for (int i = 0; i < TAPS; ++i) {      // four channels' weights lie side by side
+    const float4 v = *reinterpret_cast<const float4*>(w + (size_t)c * TAPS + 4 * i);
+    wt[4 * i] = v.x; wt[4 * i + 1] = v.y; wt[4 * i + 2] = v.z; wt[4 * i + 3] = v.w;
+  }
+  const float4 b4 = *reinterpret_cast<const float4*>(bias + c);
+  acc[0] = b4.x; acc[1] = b4.y; acc[2] = b4.z; acc[3] = b4.w;
+  const T* ur = u + (size_t)b * u_stride + c;
+#pragma unroll
+  for (int e = 0; e < 4; ++e) {
+    win[TAPS - 1][e] = to_float(ur[e]);
+    if constexpr (INB) win[TAPS - 1][e] += in_bias[c + e];
+  }
+  float* tail = tails + (size_t)slots[b] * slot_stride + c;
+#pragma unroll
+  for (int j = 0; j < TAPS - 1; ++j) {
+    const float4 v = *reinterpret_cast<const float4*>(tail + (size_t)j * C);
+    win[j][0] = v.x; win[j][1] = v.y; win[j][2] = v.z; win[j][3] = v.w;
+  }
+#pragma unroll
+  for (int j = 0; j < TAPS; ++j)
+#pragma unroll
+    for (int e = 0; e < 4; ++e) acc[e] = fmaf(wt[e * TAPS + j], win[j][e], acc[e]);
+#pragma unroll
+  for (int j = 0; j < TAPS - 1; ++j)
+    *reinterpret_cast<float4*>(tail + (size_t)j * C) = make_float4(win[j + 1][0], win[j + 1][1], win[j + 1][2], win[j + 1][3]);
+#pragma unroll
+  for (int e = 0; e < 4; ++e) out[(size_t)b * C + c + e] = from_float<T>(ACT ? acc[e] / (1.f + expf(-acc[e])) : acc[e]);
 }
 
 // The gate and the norm for rows in whole chunks of 8 that lie within one head: a thread's first kGnKeep chunks stay
@@ -324,6 +388,59 @@ int xi_conv_tail(const void* u, long long u_stride, int dtype, float* tails, lon
   else
     XI_CHECK(false, "conv_tail: unknown dtype %d", dtype);
   XI_LAUNCH_CHECK("conv_tail");
+  return 0;
+}
+
+// A step in which every sequence brings one token: row b of u is sequence b's.  The result as `xi_causal_conv`'s, and the
+// tails moved on as by `xi_conv_tail`.
+int xi_conv_step(const void* u, long long u_stride, int dtype, const float* w, const float* bias, float* tails, long long slot_stride,
+                 const long long* slots, void* out, int n_seqs, int C, int taps, const float* in_bias, int act, hipStream_t stream) {
+  XI_CHECK(n_seqs >= 0 && C > 0 && taps >= 1 && u_stride >= C, "conv_step: bad sizes B=%d C=%d taps=%d", n_seqs, C, taps);
+  XI_CHECK(slot_stride >= (long long)(taps - 1) * C, "conv_step: a slot's tail is too small");
+  XI_CHECK(dtype == kF32 || dtype == kBF16, "conv_step: unknown dtype %d", dtype);
+  if (n_seqs == 0) return 0;
+  auto whole = [](const void* p) { return (reinterpret_cast<uintptr_t>(p) & 15) == 0; };
+  if (taps <= 5 && C % 4 == 0 && slot_stride % 4 == 0 && whole(w) && whole(bias) && whole(tails)) {
+    dim3 vgrid((unsigned)n_seqs, (unsigned)((C / 4 + 63) / 64));
+    XI_CHECK(vgrid.y <= 65535u, "conv_step: too many channels");
+#define XI_STEP_AB(TT, TAPS, ACT, INB)                                                                                \
+  conv_step_vec_kernel<TT, TAPS, ACT, INB><<<vgrid, 64, 0, stream>>>((const TT*)u, u_stride, w, bias, tails, slot_stride, slots, \
+                                                                     (TT*)out, C, in_bias)
+#define XI_STEP(TT, TAPS)                               \
+  do {                                                  \
+    if (act && in_bias) XI_STEP_AB(TT, TAPS, true, true); \
+    else if (act) XI_STEP_AB(TT, TAPS, true, false);    \
+    else if (in_bias) XI_STEP_AB(TT, TAPS, false, true); \
+    else XI_STEP_AB(TT, TAPS, false, false);            \
+  } while (0)
+#define XI_STEP_TAPS(TT)          \
+  switch (taps) {                 \
+    case 1: XI_STEP(TT, 1); break; \
+    case 2: XI_STEP(TT, 2); break; \
+    case 3: XI_STEP(TT, 3); break; \
+    case 4: XI_STEP(TT, 4); break; \
+    default: XI_STEP(TT, 5); break; \
+  }
+    if (dtype == kF32) {
+      XI_STEP_TAPS(float)
+    } else {
+      XI_STEP_TAPS(bf16)
+    }
+#undef XI_STEP_TAPS
+#undef XI_STEP
+#undef XI_STEP_AB
+    XI_LAUNCH_CHECK("conv_step");
+    return 0;
+  }
+  dim3 grid((unsigned)n_seqs, (unsigned)((C + 255) / 256));
+  XI_CHECK(grid.y <= 65535u, "conv_step: too many channels");
+  if (dtype == kF32)
+    conv_step_kernel<float><<<grid, 256, 0, stream>>>((const float*)u, u_stride, w, bias, tails, slot_stride, slots, (float*)out, C, taps,
+                                                      in_bias, act);
+  else
+    conv_step_kernel<bf16><<<grid, 256, 0, stream>>>((const bf16*)u, u_stride, w, bias, tails, slot_stride, slots, (bf16*)out, C, taps,
+                                                     in_bias, act);
+  XI_LAUNCH_CHECK("conv_step");
   return 0;
 }
 

@@ -7,12 +7,15 @@
 //
 // A term y is rows in either precision or a stack of float32 partial sums, added in order.  Everything is float32 but
 // the stores of `rounded` and h_k.  x null: zeros.  `rows`: only those rows are made (x, terms and past are read there).
+// A normed term and a norm may each be made in groups: the row falls into that many equal parts, each divided by its own
+// root mean square; the weight is as long as the row.
 // Every operand is read before the row is written, and no output may be an input.
 #include "common.h"
 
 namespace xi {
 
 constexpr int kJoinPlain = 3, kJoinNormed = 2, kJoinNorms = 2;
+constexpr int kJoinGroups = 256;      // most groups of a norm
 
 struct JoinTerm {
   const void* y = nullptr;
@@ -20,6 +23,7 @@ struct JoinTerm {
   const float* w = nullptr;      // normed terms
   int parts = 1, dtype = kF32;
   float eps = 0.f, factor = 1.f;
+  int groups = 1;                // normed terms
 };
 
 struct JoinArgs {
@@ -36,6 +40,7 @@ struct JoinArgs {
   float* xout;
   const float* w[kJoinNorms];
   float eps[kJoinNorms];
+  int groups[kJoinNorms];
   void* h[kJoinNorms];
   int n_norms;
   const int* rows;
@@ -91,11 +96,33 @@ static __device__ __forceinline__ float term1(const JoinTerm& t, size_t at) {
   return s;
 }
 
+// inv[g] = 1 / sqrt(mean over the row's part g of squares + eps) for `groups` equal parts of a multiple of 4 elements; a
+// thread brings the sums of squares of its pieces of 4 elements.  The order of a part's sum is fixed by the sizes alone.
+template <int NT, int MAXV>
+static __device__ __forceinline__ void group_inverses(const float (&ss)[MAXV], int nvec, int groups, float eps, float* pieces, float* inv) {
+  const int lane = threadIdx.x & (kWave - 1), per = nvec / groups;
+  __syncthreads();                 // whoever reads `pieces` or `inv` of the norm before is done
+#pragma unroll
+  for (int v = 0; v < MAXV; ++v) {
+    const int i = v * NT + threadIdx.x;
+    if (i < nvec) pieces[i] = ss[v];
+  }
+  __syncthreads();
+  for (int g = threadIdx.x / kWave; g < groups; g += NT / kWave) {
+    float s = 0.f;
+    for (int i = lane; i < per; i += kWave) s += pieces[g * per + i];
+    s = wave_sum(s);
+    if (lane == 0) inv[g] = rsqrtf(s / (float)(4 * per) + eps);
+  }
+  __syncthreads();
+}
+
 // Rows of a multiple of 4 elements, up to 4 NT MAXV: a thread keeps its pieces of the row (and of the normed terms) in
-// registers.  NN: how many terms are normed.
-template <typename TO, int NT, int MAXV, int NN>
+// registers.  NN: how many terms are normed.  GROUPED: some norm is made in groups (of a multiple of 4 elements).
+template <typename TO, int NT, int MAXV, int NN, bool GROUPED>
 __global__ __launch_bounds__(NT) void stream_join_vec_kernel(const JoinArgs A) {
   __shared__ float scratch[NT / kWave];
+  __shared__ float pieces[GROUPED ? NT * MAXV : 1], ginv[GROUPED ? kJoinGroups : 1];
   const int r = blockIdx.x;
   const int row = A.rows ? A.rows[r] : r;
   const int H = A.H, nvec = H / 4;
@@ -123,6 +150,19 @@ __global__ __launch_bounds__(NT) void stream_join_vec_kernel(const JoinArgs A) {
   }
 #pragma unroll
   for (int n = 0; n < NN; ++n) {
+    if constexpr (GROUPED) {
+      float sq[MAXV];
+#pragma unroll
+      for (int v = 0; v < MAXV; ++v) sq[v] = dot4(y[n][v]);
+      group_inverses<NT, MAXV>(sq, nvec, A.normed[n].groups, A.normed[n].eps, pieces, ginv);
+      const int per = nvec / A.normed[n].groups;
+#pragma unroll
+      for (int v = 0; v < MAXV; ++v) {
+        const int i = v * NT + threadIdx.x;
+        if (i < nvec) fma4(s[v], A.normed[n].factor, mul4(y[n][v], ginv[i / per], join_load4(A.normed[n].w + 4 * i)));
+      }
+      continue;
+    }
     const float inv = rsqrtf(block_sum<NT / kWave>(ss[n], scratch) / (float)H + A.normed[n].eps);
 #pragma unroll
     for (int v = 0; v < MAXV; ++v) {
@@ -162,6 +202,23 @@ __global__ __launch_bounds__(NT) void stream_join_vec_kernel(const JoinArgs A) {
     }
   }
   if (A.n_norms == 0) return;
+  if constexpr (GROUPED) {
+    float sq[MAXV];
+#pragma unroll
+    for (int v = 0; v < MAXV; ++v) sq[v] = dot4(s[v]);
+#pragma unroll
+    for (int k = 0; k < kJoinNorms; ++k) {
+      if (k >= A.n_norms) break;
+      group_inverses<NT, MAXV>(sq, nvec, A.groups[k], A.eps[k], pieces, ginv);
+      const int per = nvec / A.groups[k];
+#pragma unroll
+      for (int v = 0; v < MAXV; ++v) {
+        const int i = v * NT + threadIdx.x;
+        if (i < nvec) join_store4(static_cast<TO*>(A.h[k]) + obase + 4 * i, mul4(s[v], ginv[i / per], join_load4(A.w[k] + 4 * i)));
+      }
+    }
+    return;
+  }
   float us = 0.f;
 #pragma unroll
   for (int v = 0; v < MAXV; ++v) us += dot4(s[v]);          // (pieces past the row's end are zeros)
@@ -182,25 +239,31 @@ __global__ __launch_bounds__(NT) void stream_join_vec_kernel(const JoinArgs A) {
 template <typename TO>
 __global__ __launch_bounds__(256) void stream_join_kernel(const JoinArgs A) {
   __shared__ float scratch[4];
+  __shared__ float inv[kJoinNormed][kJoinGroups], ninv[kJoinNorms][kJoinGroups];
   const int r = blockIdx.x;
   const int row = A.rows ? A.rows[r] : r;
   const int H = A.H;
   const size_t base = (size_t)row * H, obase = (size_t)r * H;
-  float inv[kJoinNormed];
+  int per[kJoinNormed], nper[kJoinNorms];
   for (int n = 0; n < kJoinNormed; ++n) {
-    inv[n] = 0.f;
+    per[n] = H;
     if (n >= A.n_normed) continue;
-    float ss = 0.f;
-    for (int i = threadIdx.x; i < H; i += 256) {
-      const float v = term1(A.normed[n], base + i);
-      ss = fmaf(v, v, ss);
+    per[n] = H / A.normed[n].groups;
+    for (int g = 0; g < A.normed[n].groups; ++g) {
+      float ss = 0.f;
+      for (int i = g * per[n] + threadIdx.x; i < (g + 1) * per[n]; i += 256) {
+        const float v = term1(A.normed[n], base + i);
+        ss = fmaf(v, v, ss);
+      }
+      const float f = rsqrtf(block_sum<4>(ss, scratch) / (float)per[n] + A.normed[n].eps);
+      if (threadIdx.x == 0) inv[n][g] = f;
     }
-    inv[n] = rsqrtf(block_sum<4>(ss, scratch) / (float)H + A.normed[n].eps);
   }
+  __syncthreads();
   auto sum_at = [&](int i) {
     float s = A.x ? A.x[base + i] : 0.f;
     for (int p = 0; p < A.n_plain; ++p) s = fmaf(A.plain[p].factor, term1(A.plain[p], base + i), s);
-    for (int n = 0; n < A.n_normed; ++n) s = fmaf(A.normed[n].factor, term1(A.normed[n], base + i) * inv[n] * A.normed[n].w[i], s);
+    for (int n = 0; n < A.n_normed; ++n) s = fmaf(A.normed[n].factor, term1(A.normed[n], base + i) * inv[n][i / per[n]] * A.normed[n].w[i], s);
     return s;
   };
   auto average_at = [&](int i, float s) {
@@ -219,11 +282,26 @@ __global__ __launch_bounds__(256) void stream_join_kernel(const JoinArgs A) {
   }
   if (A.n_norms == 0) return;
   const float mean = block_sum<4>(us, scratch) / (float)H;
-  float ninv[kJoinNorms];
-  for (int k = 0; k < kJoinNorms; ++k) ninv[k] = k < A.n_norms ? rsqrtf(mean + A.eps[k]) : 0.f;
+  for (int k = 0; k < A.n_norms; ++k) {
+    nper[k] = H / A.groups[k];
+    for (int g = 0; g < A.groups[k]; ++g) {
+      float m = mean;
+      if (A.groups[k] > 1) {
+        float gs = 0.f;
+        for (int i = g * nper[k] + threadIdx.x; i < (g + 1) * nper[k]; i += 256) {
+          const float u = average_at(i, sum_at(i));
+          gs = fmaf(u, u, gs);
+        }
+        m = block_sum<4>(gs, scratch) / (float)nper[k];
+      }
+      if (threadIdx.x == 0) ninv[k][g] = rsqrtf(m + A.eps[k]);
+    }
+  }
+  __syncthreads();
   for (int i = threadIdx.x; i < H; i += 256) {
     const float u = average_at(i, sum_at(i));
-    for (int k = 0; k < A.n_norms; ++k) static_cast<TO*>(A.h[k])[obase + i] = from_float<TO>(u * ninv[k] * A.w[k][i]);
+    for (int k = 0; k < A.n_norms; ++k)
+      static_cast<TO*>(A.h[k])[obase + i] = from_float<TO>(u * ninv[k][i / nper[k]] * A.w[k][i]);
   }
 }
 
@@ -271,11 +349,19 @@ __global__ __launch_bounds__(NT) void embed_norm_vec_kernel(const T* __restrict_
 template <typename TO>
 static void launch_join(const JoinArgs& A, int n, hipStream_t stream, bool aligned) {
   const int H = A.H;
-#define XI_JOIN_N(NT, MAXV)                                                                              \
+  bool grouped = false;
+  for (int k = 0; k < A.n_normed; ++k) grouped = grouped || A.normed[k].groups > 1;
+  for (int k = 0; k < A.n_norms; ++k) grouped = grouped || A.groups[k] > 1;
+#define XI_JOIN_G(NT, MAXV, GR)                                                                          \
   do {                                                                                                   \
-    if (A.n_normed == 0) stream_join_vec_kernel<TO, NT, MAXV, 0><<<n, NT, 0, stream>>>(A);               \
-    else if (A.n_normed == 1) stream_join_vec_kernel<TO, NT, MAXV, 1><<<n, NT, 0, stream>>>(A);          \
-    else stream_join_vec_kernel<TO, NT, MAXV, 2><<<n, NT, 0, stream>>>(A);                               \
+    if (A.n_normed == 0) stream_join_vec_kernel<TO, NT, MAXV, 0, GR><<<n, NT, 0, stream>>>(A);           \
+    else if (A.n_normed == 1) stream_join_vec_kernel<TO, NT, MAXV, 1, GR><<<n, NT, 0, stream>>>(A);      \
+    else stream_join_vec_kernel<TO, NT, MAXV, 2, GR><<<n, NT, 0, stream>>>(A);                           \
+  } while (0)
+#define XI_JOIN_N(NT, MAXV)                     \
+  do {                                          \
+    if (grouped) XI_JOIN_G(NT, MAXV, true);     \
+    else XI_JOIN_G(NT, MAXV, false);            \
   } while (0)
   if (!aligned || H > 16384) {
     stream_join_kernel<TO><<<n, 256, 0, stream>>>(A);
@@ -291,6 +377,7 @@ static void launch_join(const JoinArgs& A, int n, hipStream_t stream, bool align
     else XI_JOIN_N(1024, 4);
   }
 #undef XI_JOIN_N
+#undef XI_JOIN_G
 }
 
 }  // namespace xi
@@ -300,12 +387,13 @@ using namespace xi;
 extern "C" {
 
 // Terms in arrays of length n_terms: y[k] rows [*, H] in dtype[k] (a stack of parts[k] float32 partial sums part_stride
-// elements apart if parts[k] > 1), weight[k] float32 [H] (null: a plain term), eps[k], factor[k].  At most 3 plain and 2 normed.
+// elements apart if parts[k] > 1), weight[k] float32 [H] (null: a plain term), eps[k], factor[k], groups[k].  At most 3 plain and
+// 2 normed.  norm_groups[k]: the groups of norm k.
 // first float32 rows or null; past: n_past results past_stride elements apart; coef float32 [n_past + 2].
 int xi_stream_join(const float* x, int n_terms, const void* const* y, const int* dtype, const int* parts, long long part_stride,
-                   const float* const* weight, const float* eps, const float* factor, float* result, void* rounded,
+                   const float* const* weight, const float* eps, const float* factor, const int* groups, float* result, void* rounded,
                    const float* first, const float* past, long long past_stride, int n_past, const float* coef, float* xout,
-                   int n_norms, const float* const* norm_w, const float* norm_eps, void* const* norm_out, int out_dtype,
+                   int n_norms, const float* const* norm_w, const float* norm_eps, const int* norm_groups, void* const* norm_out, int out_dtype,
                    const int* rows, int n, int H, hipStream_t stream) {
   XI_CHECK(n >= 0 && H > 0 && n_terms >= 0 && n_norms >= 0 && n_norms <= kJoinNorms, "stream_join: bad sizes n=%d H=%d terms=%d norms=%d",
            n, H, n_terms, n_norms);
@@ -334,6 +422,9 @@ int xi_stream_join(const float* x, int n_terms, const void* const* y, const int*
     whole(t.w, 16);
     if (parts[k] > 1 && part_stride % 4) aligned = false;
     if (t.w) {
+      t.groups = groups[k];
+      XI_CHECK(t.groups >= 1 && t.groups <= kJoinGroups && H % t.groups == 0, "stream_join: rows of %d in %d groups", H, t.groups);
+      if (t.groups > 1 && (H / t.groups) % 4) aligned = false;
       XI_CHECK(A.n_normed < kJoinNormed, "stream_join: more than %d normed terms", kJoinNormed);
       A.normed[A.n_normed++] = t;
     } else {
@@ -360,6 +451,9 @@ int xi_stream_join(const float* x, int n_terms, const void* const* y, const int*
     XI_CHECK(norm_w[k] && norm_out[k], "stream_join: norm %d without a weight or a place", k);
     A.w[k] = norm_w[k];
     A.eps[k] = norm_eps[k];
+    A.groups[k] = norm_groups[k];
+    XI_CHECK(A.groups[k] >= 1 && A.groups[k] <= kJoinGroups && H % A.groups[k] == 0, "stream_join: rows of %d in %d groups", H, A.groups[k]);
+    if (A.groups[k] > 1 && (H / A.groups[k]) % 4) aligned = false;
     A.h[k] = norm_out[k];
     whole(norm_w[k], 16);
     whole(norm_out[k], ob);

@@ -634,14 +634,16 @@ def qkv_rows(qkv: torch.Tensor, q_weight: Optional[torch.Tensor], k_weight: Opti
 
 
 def moe_route(x: torch.Tensor, router: torch.Tensor, bias: Optional[torch.Tensor], top: int, all_scores: bool = False,
-              extra_rows: int = 0, sigmoid: bool = False):
+              extra_rows: int = 0, sigmoid: bool = False, correction: Optional[torch.Tensor] = None):
     """Router of a mixture of experts: z = router @ x + bias in float32 (router float32 [E, H]), the `top`
     largest (ties: the lower index), weights = softmax over the chosen logits, or with `all_scores` the
     softmax over all experts, the chosen scores divided by their sum + 1e-20.  Returns
     (idx int32 [T, top], weights float32 [T, top]), the chosen in descending order of their logits.
     `extra_rows` X > 0: the router's last X rows are no experts but further float32 products of the same
-    rows (a shared branch's gate); their results come back as a third value, float32 [T, X]."""
-    _dev(x, router, bias)
+    rows (a shared branch's gate); their results come back as a third value, float32 [T, X].
+    `correction` float32 [E] (with `all_scores` or `sigmoid`): the experts are chosen by score + correction and weighted by
+    the score without it; the chosen come in descending order of the corrected scores."""
+    _dev(x, router, bias, correction)
     X = int(extra_rows)
     if X < 0 or X >= router.shape[0]:
         raise KernelError(f"moe_route: {X} further rows of a router of {router.shape[0]}")
@@ -656,11 +658,15 @@ def moe_route(x: torch.Tensor, router: torch.Tensor, bias: Optional[torch.Tensor
             raise KernelError(f"moe_route: bias {tuple(bias.shape)} is not [{E}]")
     if not (0 < top <= min(E, 64)) or E > 1024:
         raise KernelError(f"moe_route: {top} of {E} experts (at most 64 of 1024)")
+    if correction is not None:
+        _want(correction, torch.float32, "moe_route: correction")
+        if correction.shape != (E,) or not (all_scores or sigmoid):
+            raise KernelError(f"moe_route: a correction [{E}] of scores over all experts, not {tuple(correction.shape)}")
     idx = torch.empty((T, top), dtype=torch.int32, device=x.device)
     wt = torch.empty((T, top), dtype=torch.float32, device=x.device)
     extra = torch.empty((T, X), dtype=torch.float32, device=x.device) if X else None
     _ok(lib().xi_moe_route(_p(x), _code(x, "moe_route"), _p(router), _p(bias), _p(idx), _p(wt), T, H, E, int(top),
-                           2 if sigmoid else int(bool(all_scores)), _p(extra), X, _stream()))
+                           2 if sigmoid else int(bool(all_scores)), _p(extra), X, _p(correction), _stream()))
     return (idx, wt, extra) if X else (idx, wt)
 
 
@@ -680,13 +686,14 @@ MOE_LIBRARY_ROWS = 64     # rows an expert on average from which a step of porti
 
 
 def moe_experts_library(x: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor, idx: torch.Tensor, wt: torch.Tensor,
-                        act: str = "silu", gated: bool = True, weigh_input: bool = False) -> torch.Tensor:
+                        act: str = "silu", gated: bool = True, weigh_input: bool = False, identity: int = 0,
+                        add: Optional[torch.Tensor] = None) -> torch.Tensor:
     """`moe_experts` for steps of many tokens in bfloat16: the pairs sorted by expert on the device, the rows
     gathered in that order, and one plain product of the vendor library an expert and projection (as the
     dense feed-forward's products of many rows go to the library); the hand-written kernels do the sort,
     the activation and the combine.  Reads the experts' row counts on the host: for steps that bring
-    portions, which are never recorded into a graph.  `weigh_input`: see `moe_experts` (gated experts)."""
-    _dev(x, gate_up, down, idx, wt)
+    portions, which are never recorded into a graph.  `weigh_input`, `identity`, `add`: see `moe_experts` (gated experts)."""
+    _dev(x, gate_up, down, idx, wt, add)
     T, H = x.shape
     E, F2, _ = gate_up.shape
     F, top = (F2 // 2 if gated else F2), int(idx.shape[1])
@@ -698,11 +705,12 @@ def moe_experts_library(x: torch.Tensor, gate_up: torch.Tensor, down: torch.Tens
         raise KernelError("moe_experts_library: x [T, H], gate_up [E, 2F, H] (up alone: [E, F, H]), down [E, H, F], idx and weights [T, top]")
     _want(idx, torch.int32, "moe_experts_library: idx")
     _want(wt, torch.float32, "moe_experts_library: weights")
+    _moe_rows(x, add, identity, weigh_input)
     P = T * top
     most = int(lib().xi_moe_tiles_most(P, E, 128))
     ints = torch.empty((2 * P + 3 * most + 1,), dtype=torch.int32, device=x.device)
     order, slot_of = ints[:P], ints[P:2 * P]
-    _ok(lib().xi_moe_sort(_p(idx), P, E, 128, _p(order), _p(slot_of), _p(ints[2 * P:2 * P + most]),
+    _ok(lib().xi_moe_sort(_p(idx), P, E, int(identity), 128, _p(order), _p(slot_of), _p(ints[2 * P:2 * P + most]),
                           _p(ints[2 * P + most:2 * P + 2 * most]), _p(ints[2 * P + 2 * most:2 * P + 3 * most]),
                           _p(ints[2 * P + 3 * most:]), _stream()))
     if weigh_input and not gated:
@@ -710,7 +718,7 @@ def moe_experts_library(x: torch.Tensor, gate_up: torch.Tensor, down: torch.Tens
     wt_in = wt.reshape(-1).contiguous() if weigh_input else None
     if weigh_input:
         wt = torch.ones_like(wt)
-    counts = torch.bincount(idx.reshape(-1), minlength=E).tolist()          # the one read on the host
+    counts = torch.bincount(idx.reshape(-1), minlength=E + int(identity)).tolist()          # the one read on the host
     rows = x.index_select(0, torch.div(order, top, rounding_mode="floor"))
     y = torch.empty((P, H), dtype=torch.float32, device=x.device)
     at = 0
@@ -724,13 +732,21 @@ def moe_experts_library(x: torch.Tensor, gate_up: torch.Tensor, down: torch.Tens
             torch.mm(mid, down[e].t(), out_dtype=torch.float32, out=y[at:at + n])
             at += n
     out = torch.empty((T, H), dtype=torch.float32, device=x.device)
-    _ok(lib().xi_moe_combine(_p(y), _p(slot_of), _p(wt), _p(out), T, H, top, _stream()))
+    _ok(lib().xi_moe_combine(_p(y), _p(slot_of), _p(wt), _p(out), T, H, top, _p(idx), E, _p(x if identity else None), _p(add), _stream()))
     return out
+
+
+def _moe_rows(x: torch.Tensor, add: Optional[torch.Tensor], identity: int, weigh_input: bool) -> None:
+    if add is not None and (add.shape != x.shape or add.dtype != x.dtype):
+        raise KernelError(f"moe_experts: the rows to add {tuple(add.shape)} {add.dtype} must be {tuple(x.shape)} {x.dtype}")
+    if int(identity) < 0 or (identity and weigh_input):
+        raise KernelError("moe_experts: identity experts come with weights on the experts' outputs")
 
 
 def moe_experts(x: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor, idx: torch.Tensor, wt: torch.Tensor,
                 act: str = "silu", grouped: Optional[bool] = None, tile_rows: Optional[int] = None,
-                gated: bool = True, weigh_input: bool = False) -> torch.Tensor:
+                gated: bool = True, weigh_input: bool = False, identity: int = 0,
+                add: Optional[torch.Tensor] = None) -> torch.Tensor:
     """sum over a token's chosen experts e (in the order of `idx`) of wt * down[e] @ (act(gate[e] @ x) * (up[e] @ x)):
     gate_up [E, 2F, H] (gate rows first), down [E, H, F], idx int32 / wt float32 [T, top].  Float32 [T, H].
     `gated` False: experts without a gate, wt * down[e] @ act(up[e] @ x), `gate_up` the up rows alone [E, F, H].
@@ -738,8 +754,12 @@ def moe_experts(x: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor, idx:
     float32 path and of steps with few tokens.  `grouped` (None: chosen by `moe_grouped_takes`): the pairs
     sorted by expert on the device and each expert's rows multiplied in tiles on the matrix cores.
     `weigh_input`: the weight multiplies the expert's input instead of its output, sum of expert_e(wt * x): it goes
-    onto the float32 sums of the gate and up products, before the activation."""
-    _dev(x, gate_up, down, idx, wt)
+    onto the float32 sums of the gate and up products, before the activation.
+    `identity` I: experts numbered E .. E + I - 1 have no tensors and return x itself.  `add` [T, H] in x's type: added to
+    the sum (a shared branch's result)."""
+    _dev(x, gate_up, down, idx, wt, add)
+    _moe_rows(x, add, identity, weigh_input)
+    same = x if identity else None
     acts = ACTIVATIONS if gated else UNGATED_ACTIVATIONS
     if act not in acts:
         raise KernelError(f"moe_experts: unknown activation {act!r}")
@@ -776,20 +796,20 @@ def moe_experts(x: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor, idx:
         order, slot_of = ints[:P], ints[P:2 * P]
         t_e, t_r0, t_n, n_tiles = (ints[2 * P:2 * P + most], ints[2 * P + most:2 * P + 2 * most],
                                    ints[2 * P + 2 * most:2 * P + 3 * most], ints[2 * P + 3 * most:])
-        _ok(lib().xi_moe_sort(_p(idx), P, E, bm, _p(order), _p(slot_of), _p(t_e), _p(t_r0), _p(t_n), _p(n_tiles), _stream()))
+        _ok(lib().xi_moe_sort(_p(idx), P, E, int(identity), bm, _p(order), _p(slot_of), _p(t_e), _p(t_r0), _p(t_n), _p(n_tiles), _stream()))
         mid = torch.empty((P, F), dtype=torch.bfloat16, device=x.device)
         _ok(lib().xi_moe_group(_p(x), _p(order), top, _p(gate_up), _p(t_e), _p(t_r0), _p(t_n), _p(n_tiles), most, _p(mid),
                                F, H, bm, 1 if gated else 2, acts[act], _p(wt_in), _stream()))
         y = torch.empty((P, H), dtype=torch.float32, device=x.device)
         _ok(lib().xi_moe_group(_p(mid), _p(order), top, _p(down), _p(t_e), _p(t_r0), _p(t_n), _p(n_tiles), most, _p(y),
                                H, F, bm, 0, 0, None, _stream()))
-        _ok(lib().xi_moe_combine(_p(y), _p(slot_of), _p(wt), _p(out), T, H, top, _stream()))
+        _ok(lib().xi_moe_combine(_p(y), _p(slot_of), _p(wt), _p(out), T, H, top, _p(idx), E, _p(same), _p(add), _stream()))
         return out
     mid = torch.empty((T * top, F), dtype=x.dtype, device=x.device)
     code = _code(x, "moe_experts")
     _ok(lib().xi_moe_gate_up(_p(x), _p(gate_up), _p(idx), _p(mid), code, acts[act], int(bool(gated)), T, H, F, E, top, _p(wt_in),
                              _stream()))
-    _ok(lib().xi_moe_down(_p(mid), _p(down), _p(idx), _p(wt), _p(out), code, T, H, F, E, top, _stream()))
+    _ok(lib().xi_moe_down(_p(mid), _p(down), _p(idx), _p(wt), _p(out), code, T, H, F, E, top, _p(same), _p(add), _stream()))
     return out
 
 
@@ -845,7 +865,7 @@ def qk_norm_rope_kv(qkv: torch.Tensor, q_weight: Optional[torch.Tensor],
         _p(qkv), _code(q_out, "qk_norm_rope_kv"), slices, _p(bias), _p(q_weight), _p(k_weight), ctypes.c_float(eps),
         _p(cos), _p(sin), int(rotary_dim), int(bool(interleaved)), _p(positions), _p(slots),
         _p(q_out), _p(k_cache), _p(v_cache), int(k_cache.shape[2]), T, nq, nkv, d, d,
-        int(bool(v_grouped)), int(vector_min_tokens), _stream()))
+        int(bool(v_grouped)), int(vector_min_tokens), ctypes.c_longlong(0), -1, _p(None), _p(None), _stream()))
     return q_out
 
 
@@ -1875,16 +1895,31 @@ def head_rows(qkv: torch.Tensor, slots: torch.Tensor, k_cache: torch.Tensor, v_c
               sin: Optional[torch.Tensor] = None, rotary_dim: int = 0, interleaved: bool = False,
               positions: Optional[torch.Tensor] = None, unit_norm: bool = False, eps: float = 0.0,
               bias: Optional[torch.Tensor] = None, q_weight: Optional[torch.Tensor] = None,
-              k_weight: Optional[torch.Tensor] = None) -> torch.Tensor:
+              k_weight: Optional[torch.Tensor] = None, values_in_keys: bool = False, v_cos: Optional[torch.Tensor] = None,
+              v_sin: Optional[torch.Tensor] = None) -> torch.Tensor:
     """A packed projection [T, nq d + nkv d + nkv dv]: `bias` (float32, one number a column) is added, every q and k head
     is divided by its root mean square over d and multiplied by `q_weight` / `k_weight` (float32 [d]; none: not), the first `rotary_dim` dims of every q and k head turn by the
     token's position (pairs (2i, 2i + 1) if `interleaved`, else (i, i + r / 2); `cos` / `sin` float32 [positions, r / 2]),
     then, with `unit_norm`, each head is divided by its root mean square over d (eps inside the root); k and v go into
-    the paged cache at `slots`.  Returns q [T, nq, d]."""
-    _dev(qkv, slots, k_cache, v_cache, cos, sin, positions, bias, q_weight, k_weight)
+    the paged cache at `slots`.  Returns q [T, nq, d].
+    `values_in_keys` (dv = d, no bias): the row ends with the keys, and the values are the keys as projected, before norm and
+    rotation.  `v_cos` / `v_sin` float32 [positions, dv / 2]: every value head turns by its position over all its dims, in
+    the keys' layout of pairs, and is cached so.  Rows may be columns of a longer packed row."""
+    _dev(slots, k_cache, v_cache, cos, sin, positions, bias, q_weight, k_weight, v_cos, v_sin)
     nq, nkv, d, dv, rot = int(num_heads), int(num_kv_heads), int(head_dim), int(value_dim), int(rotary_dim)
-    if qkv.dim() != 2 or qkv.shape[1] != nq * d + nkv * d + nkv * dv:
-        raise KernelError(f"head_rows: qkv {tuple(qkv.shape)} is not [T, {nq * d + nkv * d + nkv * dv}]")
+    stride = _columns(qkv, (nq + nkv) * d + (0 if values_in_keys else nkv * dv), "head_rows: qkv")
+    v_col = nq * d if values_in_keys else (nq + nkv) * d
+    if values_in_keys and (dv != d or bias is not None):
+        raise KernelError("head_rows: values that are the keys have the keys' size and no bias")
+    if v_cos is not None:
+        for t_ in (v_cos, v_sin, positions):
+            if t_ is None:
+                raise KernelError("head_rows: turned values need both tables and the positions")
+        _want(v_cos, torch.float32, "head_rows: v_cos")
+        _want(v_sin, torch.float32, "head_rows: v_sin")
+        _want(positions, torch.int32, "head_rows: positions")
+        if dv % 2 or v_cos.shape != v_sin.shape or v_cos.dim() != 2 or v_cos.shape[1] != dv // 2 or positions.shape != (qkv.shape[0],):
+            raise KernelError(f"head_rows: the values' tables must be [positions, {dv // 2}], positions [T]")
     T = qkv.shape[0]
     _want(slots, torch.int64, "head_rows: slots")
     if slots.shape != (T,) or d > 1024:
@@ -1907,19 +1942,50 @@ def head_rows(qkv: torch.Tensor, slots: torch.Tensor, k_cache: torch.Tensor, v_c
                 raise KernelError(f"head_rows: a bias or weight of {tuple(w.shape)} is not [{n}]")
     q_out = torch.empty((T, nq, d), dtype=qkv.dtype, device=qkv.device)
     if (qkv.dtype == torch.bfloat16 and v_grouped and not unit_norm and T >= HEAD_ROWS_VECTOR and d % 8 == 0 and dv % 8 == 0
-            and max(d, dv) <= 256 and (interleaved or rot % 16 == 0) and positions is not None):
+            and max(d, dv) <= 256 and (interleaved or rot % 16 == 0) and positions is not None and stride % 8 == 0
+            and (v_cos is None or (dv % 16 == 0 and not interleaved)) and qkv.data_ptr() % 16 == 0):
         # many tokens: the vectorized form of `qk_norm_rope_kv`
         none = _p(None)
         _ok(lib().xi_qk_norm_rope_kv(
             _p(qkv), BF16, 0, _p(bias), _p(q_weight), _p(k_weight), ctypes.c_float(eps), _p(cos) if rot else none, _p(sin) if rot else none,
             rot, int(bool(interleaved)), _p(positions), _p(slots), _p(q_out), _p(k_cache), _p(v_cache),
-            int(k_cache.shape[2]), T, nq, nkv, d, dv, 1, HEAD_ROWS_VECTOR, _stream()))
+            int(k_cache.shape[2]), T, nq, nkv, d, dv, 1, HEAD_ROWS_VECTOR, ctypes.c_longlong(stride), v_col, _p(v_cos), _p(v_sin), _stream()))
         return q_out
     _ok(lib().xi_head_rows(_p(qkv), _code(qkv, "head_rows"), _p(slots), _p(q_out), _p(k_cache), _p(v_cache),
                            int(k_cache.shape[2]), T, nq, nkv, d, dv, int(bool(v_grouped)), _p(cos if rot else None),
                            _p(sin if rot else None), rot, int(bool(interleaved)), _p(positions if rot else None),
-                           int(bool(unit_norm)), ctypes.c_float(eps), _p(bias), _p(q_weight), _p(k_weight), _stream()))
+                           int(bool(unit_norm)), ctypes.c_float(eps), _p(bias), _p(q_weight), _p(k_weight), ctypes.c_longlong(stride),
+                           v_col, _p(v_cos), _p(v_sin), _stream()))
     return q_out
+
+
+def head_finish_(x: torch.Tensor, heads: int, gate: Optional[torch.Tensor] = None, cos: Optional[torch.Tensor] = None,
+                 sin: Optional[torch.Tensor] = None, interleaved: bool = False, positions: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """An attention's result x [T, H dv] in place: with `cos` / `sin` (float32 [positions, dv / 2]) every head turns BACK by its
+    token's position (pairs (i, i + dv / 2), or (2i, 2i + 1) if `interleaved`); with `gate` [T, H dv] (may be columns of a
+    packed projection, in x's type) every element is then multiplied by sigmoid(gate)."""
+    _dev(x, cos, sin, positions)
+    H = int(heads)
+    if x.dim() != 2 or x.shape[1] % H or (gate is None and cos is None):
+        raise KernelError(f"head_finish: x {tuple(x.shape)} is not [T, {H} dv], or there is nothing to do")
+    T, W = x.shape
+    dv = W // H
+    gs = 0
+    if gate is not None:
+        gs = _columns(gate, W, "head_finish: gate")
+        if gate.shape[0] != T or gate.dtype != x.dtype or gate.device != x.device:
+            raise KernelError("head_finish: the gate must be rows of the same tokens in x's type")
+    if (cos is None) != (sin is None):
+        raise KernelError("head_finish: cos and sin come together")
+    if cos is not None:
+        _want(cos, torch.float32, "head_finish: cos")
+        _want(sin, torch.float32, "head_finish: sin")
+        if positions is None or dv % 2 or cos.dim() != 2 or cos.shape[1] != dv // 2 or cos.shape != sin.shape or positions.shape != (T,):
+            raise KernelError(f"head_finish: tables [positions, {dv // 2}] and positions [T] expected")
+        _want(positions, torch.int32, "head_finish: positions")
+    _ok(lib().xi_head_finish(_p(x), _code(x, "head_finish"), _p(gate), ctypes.c_longlong(gs), _p(cos), _p(sin), _p(positions),
+                             int(bool(interleaved)), T, H, dv, _stream()))
+    return x
 
 
 # ---- attention over a latent ---------------------------------------------------------------------------------
@@ -2051,6 +2117,33 @@ def conv_tail(u: torch.Tensor, tails: torch.Tensor, state_slots: torch.Tensor, c
     stride = int(tails.stride(0)) if tails.shape[0] > 1 else (taps - 1) * C
     _ok(lib().xi_conv_tail(_p(u), ctypes.c_longlong(us), _code(u, "conv_tail"), _p(tails), ctypes.c_longlong(stride),
                            _p(state_slots), _p(cu_q), B, C, taps, _p(in_bias), _stream()))
+
+
+def conv_step(u: torch.Tensor, weight: torch.Tensor, bias: torch.Tensor, tails: torch.Tensor, state_slots: torch.Tensor,
+              in_bias: Optional[torch.Tensor] = None, act: str = "silu") -> torch.Tensor:
+    """`causal_conv` and then `conv_tail` in one launch, for a step in which every sequence brings one token (row b of u is
+    sequence b's)."""
+    _dev(weight, bias, state_slots, in_bias)
+    B, C = u.shape
+    us = _columns(u, C, "conv_step: u")
+    _want(weight, torch.float32, "conv_step: weight")
+    _want(bias, torch.float32, "conv_step: bias")
+    _want(tails, torch.float32, "conv_step: tails")
+    _want(state_slots, torch.int64, "conv_step: state_slots")
+    taps = int(weight.shape[1]) if weight.dim() == 2 else 0
+    if weight.dim() != 2 or weight.shape[0] != C or taps < 1 or bias.shape != (C,) or state_slots.shape != (B,):
+        raise KernelError(f"conv_step: weight [{C}, taps], bias [{C}], a slot for each of the {B} rows")
+    if (tails.dim() != 3 or tuple(tails.shape[1:]) != (taps - 1, C) or not tails.is_cuda or tails.device != u.device
+            or (taps > 1 and tails[0].stride() != (C, 1))):
+        raise KernelError(f"conv_step: tails {tuple(tails.shape)} must be [slots, {taps - 1}, {C}] with whole slots")
+    _conv_in_bias(in_bias, C, "conv_step")
+    if act not in ("silu", "none"):
+        raise KernelError(f"conv_step: unknown activation {act!r}")
+    out = torch.empty((B, C), dtype=u.dtype, device=u.device)
+    stride = int(tails.stride(0)) if tails.shape[0] > 1 else (taps - 1) * C
+    _ok(lib().xi_conv_step(_p(u), ctypes.c_longlong(us), _code(u, "conv_step"), _p(weight), _p(bias), _p(tails), ctypes.c_longlong(stride),
+                           _p(state_slots), _p(out), B, C, taps, _p(in_bias), int(act == "silu"), _stream()))
+    return out
 
 
 def gated_group_norm(y: torch.Tensor, x: torch.Tensor, skip: torch.Tensor, z: torch.Tensor, weight: torch.Tensor, eps: float,
@@ -2365,11 +2458,11 @@ JOIN_PLAIN, JOIN_NORMED, JOIN_NORMS = 3, 2, 2         # terms without and with a
 def stream_join(x: Optional[torch.Tensor], terms=(), norms=(), out_dtype: torch.dtype = torch.float32,
                 keep: bool = False, result: Optional[torch.Tensor] = None, rounded: bool = False, average=None,
                 rows: Optional[torch.Tensor] = None, shape=None):
-    """s = x + sum over `terms` (y, weight, eps, factor) of factor * y, a term with a weight (float32 [H]) as factor * (y /
-    sqrt(mean(y^2) + eps)) * weight; y rows [T, H] in either precision or a stack [P, T, H] of float32 partial sums.  With
+    """s = x + sum over `terms` (y, weight, eps, factor[, groups]) of factor * y, a term with a weight (float32 [H]) as factor * (y /
+    sqrt(mean(y^2) + eps)) * weight (`groups`: in that many equal parts, each by its own mean); y rows [T, H] in either precision or a stack [P, T, H] of float32 partial sums.  With
     `average` = (first [T, H], past [N, T, H], n, coef [n + 2]): u = coef[0] first + sum_(j < n) coef[1 + j] past[j] + coef[n +
     1] s, else u = s.  Returns (s or None, s rounded to out_dtype or None, u or None, [u / sqrt(mean(u^2) + eps) * weight in
-    out_dtype for the (weight, eps) of `norms`]).  `keep`: s is wanted (in `result`, a float32 [T, H] that is no operand, if
+    out_dtype for the (weight, eps[, groups]) of `norms`]).  `keep`: s is wanted (in `result`, a float32 [T, H] that is no operand, if
     given); `rounded`: its rounding is; u comes back where there is an average and no `rows`.  `rows` int32: only those
     rows are made, and only the norms.  x None (with `shape` = (T, H)): zeros."""
     terms, norms = list(terms), list(norms)
@@ -2386,7 +2479,7 @@ def stream_join(x: Optional[torch.Tensor], terms=(), norms=(), out_dtype: torch.
     _dev(x, rows, result, *(t[0] for t in terms), *(t[1] for t in terms), *(n[0] for n in norms))
     stride = 0
     ys, codes, parts = [], [], []
-    for y, w, _, _ in terms:
+    for y, w, *_ in terms:
         p = 1
         if y.dim() == 3:
             _want(y, torch.float32, "stream_join: partial sums")
@@ -2420,13 +2513,16 @@ def stream_join(x: Optional[torch.Tensor], terms=(), norms=(), out_dtype: torch.
     u = torch.empty((T, H), dtype=torch.float32, device=dev) if average is not None and rows is None else None
     outs = [torch.empty((n, H), dtype=out_dtype, device=dev) for _ in norms]
     k = len(terms)
+    t_groups, n_groups = [int(t[4]) if len(t) > 4 else 1 for t in terms], [int(n[2]) if len(n) > 2 else 1 for n in norms]
+    if any(g < 1 or H % g for g in t_groups + n_groups):
+        raise KernelError(f"stream_join: rows of {H} in groups of {t_groups + n_groups}")
     voids = lambda ts: (ctypes.c_void_p * max(1, len(ts)))(*[None if t is None else t.data_ptr() for t in ts])
     floats = lambda fs: (ctypes.c_float * max(1, len(fs)))(*fs)
     ints = lambda vs: (ctypes.c_int * max(1, len(vs)))(*vs)
     _ok(lib().xi_stream_join(_p(x), k, voids(ys), ints(codes), ints(parts), ctypes.c_longlong(stride), voids([t[1] for t in terms]),
-                             floats([t[2] for t in terms]), floats([t[3] for t in terms]), _p(result), _p(low), _p(first),
+                             floats([t[2] for t in terms]), floats([t[3] for t in terms]), ints(t_groups), _p(result), _p(low), _p(first),
                              _p(past if n_past else None), ctypes.c_longlong(T * H), int(n_past), _p(coef), _p(u), len(norms),
-                             voids([w for w, _ in norms]), floats([e for _, e in norms]), voids(outs),
+                             voids([n[0] for n in norms]), floats([n[1] for n in norms]), ints(n_groups), voids(outs),
                              _CODE[out_dtype], _p(rows), n, H, _stream()))
     return result, low, u, outs
 

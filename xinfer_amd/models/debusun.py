@@ -75,9 +75,9 @@ class Rotary:
             out["scaling"] = dict(zip(("factor", "original", "fast", "slow"), self.scaling))
         return out
 
-    def spec(self, head_dim: int, max_positions: int) -> PartSpec:
+    def spec(self, head_dim: int, max_positions: int, interleaved: bool = True) -> PartSpec:
         params: Dict[str, Any] = dict(head_dim=head_dim, rotary_dim=self.dims, theta=self.base, max_positions=max_positions,
-                                      interleaved=True)
+                                      interleaved=interleaved)
         if self.scaling is not None:
             factor, original, fast, slow = self.scaling
             params["scaling"] = dict(kind="ramp", factor=factor, original=original, fast=fast, slow=slow)

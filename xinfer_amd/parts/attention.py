@@ -30,6 +30,13 @@ with `chunk` c a query at position p sees the keys p - p mod c .. p (chunks coun
 a layer the cache keeps the last c tokens, as of a window).  Values as long as the keys go through the plain form's fused kernel for the
 heads, others a head at a time (`kernels.head_rows`), and then the attention kernels that know the score's options.
 
+The general form's heads one by one (`kernels.head_rows`) also take: `values="keys"`: the values are the keys as projected,
+before norm and rotation, and there is no value product; `value_position` (a position encoding over `value_dim`): every value
+head turns by its own position and is cached so, and a query's result turns back by the query's position; `gate`: the heads
+side by side times sigmoid(W_g x), element by element, before the output product (tensor `gate` [heads * value_dim, hidden],
+packed with q, k and v).  `sinks`: one more weight in every head's denominator without a key or a value, exp(sink) with
+"learned" (tensor `sink` [heads], neither scaled nor capped) or 1 with "one" (a sink whose score is 0).
+
 A third group of options, each a parameter of the spec, goes through `_forward_rows` (no rotation, `qk_norm` "row" or
 none): `conv` n: q, k and v pass a causal convolution per channel over the last n tokens right after the
 projection (tensors `q_conv`, `k_conv`, `v_conv` [channels, n], no bias; the last n - 1 projected rows of a request are
@@ -90,14 +97,29 @@ class PagedAttention(Mixer):
         # the options that the fused q/k kernel and the attention kernels of the plain form do not know
         self.general = bool(self.dv != self.d or self.row_norm or self.softcap > 0 or self.slope_values is not None
                             or self.value_mix_key is not None or self.chunk > 0 or spec.get("general", False))
+        self.values_in_keys = spec.get("values") == "keys"
+        if spec.get("values") not in (None, "keys"):
+            raise ValueError(f"values {spec.get('values')!r}: 'keys' or none")
+        if self.values_in_keys and (self.dv != self.d or self.bias):
+            raise ValueError("values that are the keys have the keys' size and no bias")
+        self.gate = bool(spec.get("gate", False))
+        self.sink_kind = spec.get("sinks")
+        if self.sink_kind not in (None, "learned", "one"):
+            raise ValueError(f"sinks {self.sink_kind!r}: 'learned', 'one' or none")
+        self.sinks = None            # float32 [nq]
+        vpos = spec.get("value_position")
+        self.value_position = position_encoding_class(vpos.kind)(vpos, dtype) if vpos is not None else None
+        head_options = self.values_in_keys or self.gate or self.value_position is not None
+        if head_options or self.sink_kind:
+            self.general = True
         interleaved = spec.get("position") is not None and bool(spec["position"].get("interleaved", False))
         self.head_norm = self.qk_norm and not self.row_norm and not self.unit_norm          # a weight [head_dim], before the rotation
         # the general form's heads are made ready a head at a time where they are normed one by one, turned in pairs
         # (2i, 2i + 1) or have biases; else a row at a time
-        self.by_head = self.general and (self.unit_norm or self.head_norm or interleaved or self.bias)
+        self.by_head = self.general and (self.unit_norm or self.head_norm or interleaved or self.bias or head_options)
         if self.by_head and (self.row_norm or self.value_mix_key is not None):
-            raise NotImplementedError("attention whose heads are normed one by one, turned in pairs (2i, 2i + 1) or have biases "
-                                      "takes no norm over the whole projection and no blended values")
+            raise NotImplementedError("attention whose heads are normed one by one, turned in pairs (2i, 2i + 1), gated, have biases, "
+                                      "turned values or the keys for values takes no norm over the whole projection and no blended values")
         self.taps = int(spec.get("conv") or 0)
         self.value_unit = spec.get("value_norm") == "head_unit"
         if spec.get("value_norm") not in (None, "head_unit"):
@@ -109,9 +131,9 @@ class PagedAttention(Mixer):
         if self.rows_form:
             self.general = True
             if (self.by_head or spec.get("position") is not None or self.softcap > 0 or self.slope_values is not None
-                    or self.value_mix_key is not None or self.chunk > 0 or self.bias or (self.qk_norm and not self.row_norm)):
+                    or self.value_mix_key is not None or self.chunk > 0 or self.bias or self.sink_kind or (self.qk_norm and not self.row_norm)):
                 raise NotImplementedError("attention with a convolution, normed values, mixed heads or a gate a head takes the "
-                                          "q/k norm over the whole projection or none, and no rotation, cap, bias, chunks or blend")
+                                          "q/k norm over the whole projection or none, and no rotation, cap, bias, chunks, sinks or blend")
         self.conv_w = self.talk = None
         if self.general and not self.by_head and spec.get("position") is not None and self.qk_norm:
             raise NotImplementedError("a rotation and a norm over the whole projection")
@@ -126,6 +148,9 @@ class PagedAttention(Mixer):
                               and kernels.decode_attention_takes(self.nq, self.nkv, self.d))
         pos = spec.get("position")
         self.position = position_encoding_class(pos.kind)(pos, dtype) if pos is not None else None
+        if self.value_position is not None and (self.value_position.rotary_dim != self.dv or (
+                self.position is not None and self.position.interleaved != self.value_position.interleaved)):
+            raise ValueError("turned values turn over all their dims, in the keys' layout of pairs")
         self.qkv: Optional[Linear] = None
         self.o: Optional[Linear] = None
         self.q_norm_w = self.k_norm_w = None
@@ -136,7 +161,7 @@ class PagedAttention(Mixer):
              "q_bias": "q_proj.bias", "k_bias": "k_proj.bias", "v_bias": "v_proj.bias",
              "q_norm": "q_norm.weight", "k_norm": "k_norm.weight", "value_mix": "value_mix",
              "q_conv": "q_conv.weight", "k_conv": "k_conv.weight", "v_conv": "v_conv.weight", "talk": "talk",
-             "head_gate": "head_gate.weight"}
+             "head_gate": "head_gate.weight", "gate": "gate_proj.weight", "sink": "sinks"}
 
     @classmethod
     def _names(cls, spec: PartSpec, prefix: str):
@@ -149,8 +174,14 @@ class PagedAttention(Mixer):
         h, nq, nkv, d = (int(spec[k]) for k in ("hidden_size", "num_heads", "num_kv_heads", "head_dim"))
         dv = int(spec.get("value_dim") or d)
         n = cls._names(spec, prefix)
-        out = [TensorDecl(n["q"], (nq * d, h)), TensorDecl(n["k"], (nkv * d, h)),
-               TensorDecl(n["v"], (nkv * dv, h)), TensorDecl(n["o"], (h, nq * dv))]
+        out = [TensorDecl(n["q"], (nq * d, h)), TensorDecl(n["k"], (nkv * d, h))]
+        if spec.get("values") != "keys":
+            out.append(TensorDecl(n["v"], (nkv * dv, h)))
+        out.append(TensorDecl(n["o"], (h, nq * dv)))
+        if spec.get("gate", False):
+            out.append(TensorDecl(n["gate"], (nq * dv, h)))
+        if spec.get("sinks") == "learned":
+            out.append(TensorDecl(n["sink"], (nq,), "normal(0,1)"))
         if spec.get("bias", False):    # q, k and v only: the reference's o_proj has none (attention.rs:596-608)
             out += [TensorDecl(n["q_bias"], (nq * d,)), TensorDecl(n["k_bias"], (nkv * d,)),
                     TensorDecl(n["v_bias"], (nkv * dv,))]
@@ -176,7 +207,15 @@ class PagedAttention(Mixer):
             t = store.get(name, None, device)
             return t.to(self.dtype) if (self.dtype == torch.float32 or t.dtype != torch.float32) else t
         names = self._names(self.spec, prefix)
-        parts = [lin(names[n]) for n in (("q", "k", "v", "head_gate") if self.head_gate else ("q", "k", "v"))]
+        packed = ("q", "k") + (() if self.values_in_keys else ("v",)) + (("head_gate",) if self.head_gate else ()) \
+            + (("gate",) if self.gate else ())
+        parts = [lin(names[n]) for n in packed]
+        if self.sink_kind == "learned":
+            self.sinks = store.get(names["sink"], torch.float32, device).reshape(-1).contiguous()
+        elif self.sink_kind == "one":
+            self.sinks = torch.zeros(self.nq, dtype=torch.float32, device=device)
+        if self.value_position is not None:
+            self.value_position.load(store, prefix, device)
         if self.taps >= 1:
             self.conv_w = torch.cat([store.get(names[n], torch.float32, device) for n in ("q_conv", "k_conv", "v_conv")]).contiguous()
         if self.talking:
@@ -273,7 +312,7 @@ class PagedAttention(Mixer):
                 if v_other is None:
                     raise RuntimeError(f"values {self.value_mix_key!r} are blended in before the layer that makes them has run")
         pos = self.position
-        if self.by_head and self.dv == self.d <= 256 and not self.unit_norm:      # the plain form's heads under another score
+        if self.by_head and self.dv == self.d <= 256 and not self.unit_norm and not (self.values_in_keys or self.gate or self.value_position):      # the plain form's heads under another score
             q = kernels.qk_norm_rope_kv(
                 qkv, self.q_norm_w, self.k_norm_w, self.qk_norm_eps,
                 pos.cos if pos is not None else ctx.empty_f32, pos.sin if pos is not None else ctx.empty_f32,
@@ -281,25 +320,32 @@ class PagedAttention(Mixer):
                 ctx.positions, slots, cache.k, cache.v, self.nq, self.nkv, self.d, v_grouped=vt,
                 vector_min_tokens=128 if ctx.max_q_len > 1 else self.VECTOR_MIN_DECODE, bias=self.qkv_bias)
             a = kernels.attention(q, cache.k, cache.v, ctx, cache.group, self.scale, self.window, v_grouped=vt,
-                                  softcap=self.softcap, slopes=self.slopes, chunk=self.chunk)
+                                  softcap=self.softcap, slopes=self.slopes, chunk=self.chunk, sinks=self.sinks)
             return self.o(a, out_dtype=self.dtype, allow_split=True, sink=sink)
         if self.by_head:
-            q = kernels.head_rows(qkv, slots, cache.k, cache.v, self.nq, self.nkv, self.d, self.dv, v_grouped=vt,
+            heads = qkv.shape[1] - (self.nq * self.dv if self.gate else 0)
+            vpos = self.value_position
+            q = kernels.head_rows(qkv[:, :heads], slots, cache.k, cache.v, self.nq, self.nkv, self.d, self.dv, v_grouped=vt,
                                   cos=pos.cos if pos is not None else None, sin=pos.sin if pos is not None else None,
                                   rotary_dim=pos.rotary_dim if pos is not None else 0,
-                                  interleaved=pos.interleaved if pos is not None else False, positions=ctx.positions,
+                                  interleaved=any(p is not None and p.interleaved for p in (pos, vpos)), positions=ctx.positions,
                                   unit_norm=self.unit_norm, eps=self.qk_norm_eps, bias=self.qkv_bias,
                                   q_weight=self.q_norm_w if self.head_norm else None,
-                                  k_weight=self.k_norm_w if self.head_norm else None)
+                                  k_weight=self.k_norm_w if self.head_norm else None, values_in_keys=self.values_in_keys,
+                                  v_cos=vpos.cos if vpos is not None else None, v_sin=vpos.sin if vpos is not None else None)
             a = kernels.attention(q, cache.k, cache.v, ctx, cache.group, self.scale, self.window, v_grouped=vt,
-                                  softcap=self.softcap, slopes=self.slopes, chunk=self.chunk)
+                                  softcap=self.softcap, slopes=self.slopes, chunk=self.chunk, sinks=self.sinks)
+            if self.gate or vpos is not None:
+                kernels.head_finish_(a, self.nq, gate=qkv[:, heads:] if self.gate else None,
+                                     cos=vpos.cos if vpos is not None else None, sin=vpos.sin if vpos is not None else None,
+                                     interleaved=vpos.interleaved if vpos is not None else False, positions=ctx.positions)
             return self.o(a, out_dtype=self.dtype, allow_split=True, sink=sink)
         q = kernels.qkv_rows(qkv, self.q_norm_w, self.k_norm_w, self.qk_norm_eps, slots, cache.k, cache.v,
                              self.nq, self.nkv, self.d, self.dv, v_grouped=vt, v_other=v_other, mix=self.mix,
                              cos=pos.cos if pos is not None else None, sin=pos.sin if pos is not None else None,
                              rotary_dim=pos.rotary_dim if pos is not None else 0, positions=ctx.positions)
         a = kernels.attention(q, cache.k, cache.v, ctx, cache.group, self.scale, self.window, v_grouped=vt,
-                              softcap=self.softcap, slopes=self.slopes, chunk=self.chunk)
+                              softcap=self.softcap, slopes=self.slopes, chunk=self.chunk, sinks=self.sinks)
         return self.o(a, out_dtype=self.dtype, allow_split=True, sink=sink)
 
     def _forward_rows(self, x, ctx: StepContext, cache: LayerCache):

@@ -181,11 +181,12 @@ class Folded:
 @dataclass
 class Term:
     """Something the stream is to get: scale * y, or with a `weight` (float32 [H]) scale * (y / sqrt(mean(y^2) + eps)) *
-    weight.  y: rows in either precision, or a stack [P, T, H] of float32 partial sums."""
+    weight (with `groups`: in that many equal parts of the row, each divided by its own root mean square).  y: rows in either precision, or a stack [P, T, H] of float32 partial sums."""
     y: torch.Tensor
     weight: Optional[torch.Tensor] = None
     eps: float = 0.0
     scale: float = 1.0
+    groups: int = 1
 
 
 @dataclass
@@ -230,10 +231,12 @@ class Part:
     # Folding a norm into the products around it (see `Folded`): a mixer or feed-forward whose
     # `forward` takes a keyword `sink: Optional[NormSink]` says `takes_sink`; one whose `forward`
     # takes a `Folded` in place of its input rows says `takes_folded`; a norm that can be folded
-    # (a weight vector `weight` in float32, `eps`, `dim`) says `foldable`.
+    # (a weight vector `weight` in float32, `eps`, `dim`) says `foldable`.  One that the pass over an open stream can make
+    # (the same, over `groups` equal parts of the row) says `joinable`.
     takes_sink = False
     takes_folded = False
     foldable = False
+    joinable = False
 
     def __init__(self, spec: PartSpec, dtype: torch.dtype):
         self.spec = spec

@@ -15,6 +15,10 @@ the rounding of the new stream for the next sublayer are one kernel (`Norm.forwa
 "parallel": x <- x + (mixer(norm1(x)) + ff(norm2(x))), both of the same x, each with a norm of its own; a layer may have
 no feed-forward.  One pass makes x (what the layers before left to be added) and both normed rows; the two branches are
 left to be added by whoever reads the stream next (`Stream.terms`).
+
+"sandwich": x <- x + norm1b(mixer(norm1(x))); x <- x + norm2b(ff(norm2(x))): a norm before and after every sublayer; a layer
+may have no feed-forward.  A sublayer's output is left to be normed and added by the pass that makes the next norm (one pass
+over the stream a sublayer: the branch's norm, the sum, the norm of the new row).
 """
 from __future__ import annotations
 
@@ -247,3 +251,67 @@ class ParallelBlock(Block):
         if self.ffn is not None:
             terms += (Term(self.ffn.forward(rows[1], ctx)),)
         return Stream(stream.resid, terms=terms)
+
+
+@register_block("sandwich")
+class SandwichBlock(Block):
+    """`layer.norms` names, in running order, the norms before and after the mixer and those before and after the
+    feed-forward (the last two absent if the layer has none).  Norm kinds that the pass over the stream cannot make itself
+    (`parts.joining.joins`) are run one by one, on a joined stream."""
+    takes_open = True
+
+    def __init__(self, layer: LayerSpec, dtype: torch.dtype):
+        super().__init__(layer, dtype)
+        self.mixer = mixer_class(layer.mixer.kind)(layer.mixer, dtype)
+        self.ffn = (feed_forward_class(layer.feed_forward.kind)(layer.feed_forward, dtype)
+                    if layer.feed_forward is not None else None)
+        items = layer.norm_items(4 if self.ffn is not None else 2)
+        self._names = [n for n, _ in items]
+        self.norms = [norm_class(n.kind)(n, dtype) for _, n in items]
+        self.joined = all(joins(n) for n in self.norms)
+
+    @property
+    def writes_stream(self) -> bool:
+        return not self.joined
+
+    @classmethod
+    def declare(cls, layer: LayerSpec) -> List[TensorDecl]:
+        p = layer.prefix
+        out = mixer_class(layer.mixer.kind).declare(layer.mixer, f"{p}.{layer.mixer_name}")
+        if layer.feed_forward is not None:
+            out += feed_forward_class(layer.feed_forward.kind).declare(layer.feed_forward, f"{p}.{layer.feed_forward_name}")
+        for name, n in layer.norm_items(4 if layer.feed_forward is not None else 2):
+            out += norm_class(n.kind).declare(n, f"{p}.{name}")
+        return out
+
+    def load(self, store: WeightStore, device) -> None:
+        p = self.layer.prefix
+        self.mixer.load(store, f"{p}.{self.layer.mixer_name}", device)
+        if self.ffn is not None:
+            self.ffn.load(store, f"{p}.{self.layer.feed_forward_name}", device)
+        for name, norm in zip(self._names, self.norms):
+            norm.load(store, f"{p}.{name}", device)
+
+    @property
+    def graph_safe(self) -> bool:
+        return all(p.graph_safe for p in (self.mixer, *self.norms, *(() if self.ffn is None else (self.ffn,))))
+
+    def cache_need(self) -> Optional[KVNeed]:
+        return self.mixer.cache_need()
+
+    def state_need(self) -> Optional[StateNeed]:
+        return self.mixer.state_need()
+
+    def _sublayer(self, stream: Stream, before, after, run) -> Stream:
+        if self.joined:
+            stream, _, (h,) = join(stream, self.dtype, (before,))
+            return Stream(stream.resid, terms=(Term(run(h), after.weight, after.eps, groups=getattr(after, "groups", 1)),))
+        resid = join(stream, self.dtype)[0].resid
+        after.forward_branch(resid, run(before.forward(resid, None, self.dtype)), None)
+        return Stream(resid)
+
+    def forward(self, stream: Stream, ctx: StepContext, cache: LayerCache) -> Stream:
+        stream = self._sublayer(stream, self.norms[0], self.norms[1], lambda h: self.mixer.forward(h, ctx, cache))
+        if self.ffn is not None:
+            stream = self._sublayer(stream, self.norms[2], self.norms[3], lambda h: self.ffn.forward(h, ctx))
+        return stream

@@ -31,6 +31,7 @@ from ..config.spec import PartSpec
 from ..weights.store import TensorDecl, WeightStore
 from .base import LayerCache, Mixer, StateNeed, StepContext, register_mixer
 from .linear import Linear
+from .short_conv import short_conv
 
 
 class _ChannelState(Mixer):
@@ -148,12 +149,8 @@ class RealGatedRecurrence(_ChannelState):
             raise RuntimeError("a gated recurrence was given no state slots")
         w = self.width
         p = self.proj(x, out_dtype=self.dtype)
-        tails = (cache.states["conv_tail"] if self.taps > 1 else
-                 torch.empty((cache.state.shape[0], 0, w), dtype=torch.float32, device=x.device))
-        u = kernels.causal_conv(p[:, w:], self.conv_w, self.conv_b, tails, ctx.state_slots, ctx.tok_seq, ctx.cu_q,
-                                in_bias=self.x_bias, act="none")
-        if self.taps > 1:
-            kernels.conv_tail(p[:, w:], tails, ctx.state_slots, ctx.cu_q, in_bias=self.x_bias)
+        u = short_conv(p[:, w:], self.conv_w, self.conv_b, cache.states["conv_tail"] if self.taps > 1 else None, ctx,
+                       in_bias=self.x_bias, act="none")
         terms = kernels.rglru_terms(u, self.gates, self.r_bias, self.i_bias, self.rate)
         y = kernels.channel_scan(p[:, :w], "gelu_tanh", cache.state, ctx.state_slots, ctx.cu_q, ready=terms, gate_bias=self.y_bias,
                                  **self._cutting(ctx))

@@ -12,8 +12,9 @@ from .base import Norm, Stream, Term
 
 
 def joins(*norms: Norm) -> bool:
-    """Whether the pass can make these norms itself: their form is x / sqrt(mean(x^2) + eps) * weight."""
-    return len(norms) <= kernels.JOIN_NORMS and all(n.foldable for n in norms)
+    """Whether the pass can make these norms itself: their form is x / sqrt(mean(x^2) + eps) * weight, over the row or over
+    equal parts of it."""
+    return len(norms) <= kernels.JOIN_NORMS and all(n.foldable or n.joinable for n in norms)
 
 
 def join(stream: Stream, dtype: torch.dtype, norms: Sequence[Norm] = (), rounded: bool = False,
@@ -24,8 +25,8 @@ def join(stream: Stream, dtype: torch.dtype, norms: Sequence[Norm] = (), rounded
     if stream.folded is not None:
         raise RuntimeError("the stream carries a half-done norm of the block before")
     terms = () if stream.pending is None else (Term(stream.pending, scale=stream.pending_scale),)
-    terms = [(t.y, t.weight, t.eps, t.scale) for t in terms + tuple(stream.terms)]
-    weighed = [(n.weight, n.eps) for n in norms]
+    terms = [(t.y, t.weight, t.eps, t.scale, t.groups) for t in terms + tuple(stream.terms)]
+    weighed = [(n.weight, n.eps, getattr(n, "groups", 1)) for n in norms]
     x = stream.resid
     while (sum(t[1] is None for t in terms) > kernels.JOIN_PLAIN or sum(t[1] is not None for t in terms) > kernels.JOIN_NORMED):
         first = next(t for t in terms if (t[1] is None) == (sum(u[1] is None for u in terms) > kernels.JOIN_PLAIN))

@@ -16,10 +16,12 @@ weight multiply what the expert SEES, sum of expert_e(weight_e * x), instead of 
 products are linear, so the kernels put the weight on their float32 sums, before the activation); `shared` = {intermediate_size,
 activation, gated, gate}: one more expert of the same form that every token takes, added to the result,
 times sigmoid(w_g . x) with a vector w_g of its own if `gate` says so (that product rides with the
-router's, in float32).
+router's, in float32); `correction: True` (with scores "all" or "sigmoid"): a float32 tensor of one number an output is added
+to the scores where the experts are chosen, and to nothing else; `identity` I: the router's last I outputs stand for experts
+without tensors that return their input (all scores are over both kinds).
 
 Tensor names under the part's prefix (`names` of the spec replaces any of them): `router`,
-`router_bias`, and per expert i `expert{i}.gate`, `expert{i}.up`, `expert{i}.down`, in which "{i}" is
+`router_bias`, `correction`, and per expert i `expert{i}.gate`, `expert{i}.up`, `expert{i}.down`, in which "{i}" is
 the expert's number; `shared_gate`, `shared_up`, `shared_down` and `shared_open` (the vector w_g, [1, H]).
 """
 from __future__ import annotations
@@ -42,7 +44,8 @@ class RoutedExperts(FeedForward):
     NAMES = {"router": "router.weight", "router_bias": "router.bias", "gate": "experts.{i}.gate_proj.weight",
              "up": "experts.{i}.up_proj.weight", "down": "experts.{i}.down_proj.weight",
              "shared_gate": "shared_expert.gate_proj.weight", "shared_up": "shared_expert.up_proj.weight",
-             "shared_down": "shared_expert.down_proj.weight", "shared_open": "shared_expert_gate.weight"}
+             "shared_down": "shared_expert.down_proj.weight", "shared_open": "shared_expert_gate.weight",
+             "correction": "router.correction"}
 
     def __init__(self, spec: PartSpec, dtype: torch.dtype):
         super().__init__(spec, dtype)
@@ -61,8 +64,15 @@ class RoutedExperts(FeedForward):
             raise ValueError(f"weigh {spec.get('weigh')!r}: 'output' (the expert's result) or 'input'")
         if self.weigh_input and not self.gated:
             raise NotImplementedError("a weight on the experts' input is built for gated experts")
-        if not (0 < self.top <= self.experts):
-            raise ValueError(f"{self.top} of {self.experts} experts cannot be chosen")
+        self.identity = int(spec.get("identity") or 0)       # experts without tensors, behind the others
+        if self.identity < 0 or not (0 < self.top <= self.experts + self.identity):
+            raise ValueError(f"{self.top} of {self.experts} + {self.identity} experts cannot be chosen")
+        if self.identity and self.weigh_input:
+            raise NotImplementedError("identity experts with weights on the experts' inputs")
+        self.corrected = bool(spec.get("correction", False))
+        if self.corrected and not (self.all_scores or self.sigmoid_scores):
+            raise ValueError("a correction is added to scores over all experts or to sigmoids")
+        self.correction: Optional[torch.Tensor] = None   # float32 [E + I]
         sh = spec.get("shared")
         self.shared = None if not sh else dict(inter=int(sh["intermediate_size"]), act=str(sh.get("activation", self.activation)),
                                                gated=bool(sh.get("gated", self.gated)), open=bool(sh.get("gate", False)))
@@ -98,9 +108,12 @@ class RoutedExperts(FeedForward):
     def declare(cls, spec: PartSpec, prefix: str) -> List[TensorDecl]:
         h, f, e = int(spec["hidden_size"]), int(spec["intermediate_size"]), int(spec["num_experts"])
         n = cls._names(spec, prefix)
-        out = [TensorDecl(n["router"], (e, h))]
+        outputs = e + int(spec.get("identity") or 0)
+        out = [TensorDecl(n["router"], (outputs, h))]
         if spec.get("router_bias", False):
-            out.append(TensorDecl(n["router_bias"], (e,)))
+            out.append(TensorDecl(n["router_bias"], (outputs,)))
+        if spec.get("correction", False):
+            out.append(TensorDecl(n["correction"], (outputs,), "normal(0,0.05)"))
         gated = bool(spec.get("gated", True))
         for i in range(e):
             if gated:
@@ -121,6 +134,8 @@ class RoutedExperts(FeedForward):
         self.router_w = store.get(n["router"], torch.float32, device).contiguous()
         if self.router_bias:
             self.router_b = store.get(n["router_bias"], torch.float32, device).contiguous()
+        if self.corrected:
+            self.correction = store.get(n["correction"], torch.float32, device).contiguous()
         gu, dn = [], []
         for i in range(self.experts):
             u, d = (store.get(n[k].replace("{i}", str(i)), self.dtype, device) for k in ("up", "down"))
@@ -143,23 +158,25 @@ class RoutedExperts(FeedForward):
     def forward(self, x: torch.Tensor, ctx: StepContext) -> torch.Tensor:
         opens = bool(self.shared and self.shared["open"])
         routed = kernels.moe_route(x, self.router_w, self.router_b, self.top, all_scores=self.all_scores,
-                                   extra_rows=1 if opens else 0, sigmoid=self.sigmoid_scores)
+                                   extra_rows=1 if opens else 0, sigmoid=self.sigmoid_scores, correction=self.correction)
         idx, wt = routed[0], routed[1]
+        # the shared expert's result is added where the experts' are, unless a factor opens it
+        add = self._shared(x) if self.shared and not opens else None
         # a step that brings portions is never recorded: with many rows an expert it may read the experts' row
         # counts on the host and hand each expert's rows to the vendor library, as the dense products of many rows go
         if (ctx.max_q_len > 1 and x.dtype == torch.bfloat16 and self.LIBRARY
                 and x.shape[0] * self.top >= kernels.MOE_LIBRARY_ROWS * self.experts):
             out = kernels.moe_experts_library(x, self.gate_up, self.down, idx, wt, self.activation, gated=self.gated,
-                                              weigh_input=self.weigh_input)
+                                              weigh_input=self.weigh_input, identity=self.identity, add=add)
         else:
             out = kernels.moe_experts(x, self.gate_up, self.down, idx, wt, self.activation, gated=self.gated,
-                                      weigh_input=self.weigh_input)
-        if self.shared:
-            out = self._add_shared(out, x, routed[2][:, 0] if opens else None)
+                                      weigh_input=self.weigh_input, identity=self.identity, add=add)
+        if opens:            # out (float32) += sigmoid(opening) * the shared expert's result
+            out = kernels.gated_add_(out, self._shared(x), routed[2][:, 0])
         return out
 
-    def _add_shared(self, out: torch.Tensor, x: torch.Tensor, opening: Optional[torch.Tensor]) -> torch.Tensor:
-        """out (float32) += [sigmoid(opening) *] the shared expert's result for every row."""
+    def _shared(self, x: torch.Tensor) -> torch.Tensor:
+        """The shared expert's result for every row."""
         sh = self.shared
         if sh["gated"]:
             m = self.shared_up(x, out_dtype=self.dtype, gated=True, act=sh["act"])
@@ -167,7 +184,4 @@ class RoutedExperts(FeedForward):
                 m = kernels.act_mul(self.shared_up(x, out_dtype=self.dtype), sh["act"])
         else:
             m = kernels.act_(self.shared_up(x, out_dtype=self.dtype), sh["act"])
-        y = self.shared_down(m, out_dtype=self.dtype)
-        if opening is None:
-            return kernels.scaled_sum(out, y, 1.0)
-        return kernels.gated_add_(out, y, opening)
+        return self.shared_down(m, out_dtype=self.dtype)

@@ -26,6 +26,7 @@ from ..config.spec import PartSpec
 from ..weights.store import TensorDecl, WeightStore
 from .base import LayerCache, Mixer, StateNeed, StepContext, register_mixer
 from .linear import Linear
+from .short_conv import short_conv
 
 
 @register_mixer("mamba2")
@@ -89,13 +90,7 @@ class Mamba2(Mixer):
         H, dv, N, G, inner, C = self.heads, self.dv, self.n, self.groups, self.inner, self.channels
         p = self.proj(x, out_dtype=self.dtype)
         z, u, dt = p[:, :inner], p[:, inner:inner + C], p[:, inner + C:]
-        if self.taps > 1:
-            tails = cache.states["conv_tail"]
-        else:
-            tails = torch.empty((cache.state.shape[0], 0, C), dtype=torch.float32, device=x.device)
-        xbc = kernels.causal_conv(u, self.conv_w, self.conv_b, tails, ctx.state_slots, ctx.tok_seq, ctx.cu_q)
-        if self.taps > 1:
-            kernels.conv_tail(u, tails, ctx.state_slots, ctx.cu_q)
+        xbc = short_conv(u, self.conv_w, self.conv_b, cache.states["conv_tail"] if self.taps > 1 else None, ctx)
         xs, b, c = xbc[:, :inner], xbc[:, inner:inner + G * N], xbc[:, inner + G * N:]
         cut = {}
         if ctx.max_q_len > 1 and ctx.cu_q_host:
