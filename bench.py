@@ -112,9 +112,13 @@ TISOSUN_SIZES = ("1k", "4k", "2k-d")
 # taps), the linear attention's heads as Lilalorn's, half of a head turned, a token input of 256 columns a layer
 TISOSUN_SIDE = 256
 TISOSUN_TAPS = 4
+LITIZEN_SIZES = ("1k", "4k", "4k-moe")
+# Litizen's own sizes at every width: the state space as Debusun's, norms in 4 groups, 4 taps in front of every mixer, half of an
+# attention_2 head turned; with experts, 2 identity experts beside them and a shared one as wide as an expert
+LITIZEN_GROUPS, LITIZEN_TAPS, LITIZEN_IDENTITY = 4, 4, 2
 DESIGN_CHOICES = {"mufenex": (tuple(k for k in DESIGN_SIZES if "g2" not in k and k != "2k-d"), "qwen3"), "lilalorn": (LILALORN_SIZES, "mufenex"),
                   "debusun": (DEBUSUN_SIZES, "mufenex"), "vuzazen": (VUZAZEN_SIZES, "debusun"),
-                  "tisosun": (TISOSUN_SIZES, "mufenex")}
+                  "tisosun": (TISOSUN_SIZES, "mufenex"), "litizen": (LITIZEN_SIZES, "debusun")}
 DESIGN_VOCAB = 32000
 MODELS = {"0.6b": QWEN3_0_6B, "8b": QWEN3_8B, "14b": QWEN3_14B, "32b": QWEN3_32B}
 CONTEXT = 4096
@@ -252,7 +256,7 @@ def product(spec: str, dev="cuda:0") -> int:
 
 def design_compare(spec: str, layers, steps: int, warmup: int, batch: int, context: int, prefill_tokens: int,
                    family: str = "both", only: str = "all") -> int:
-    """Mufenex beside Qwen3, Lilalorn, Debusun or Tisosun beside Mufenex, or Vuzazen beside Debusun, at equal sizes: ms of the
+    """Mufenex beside Qwen3, Lilalorn, Debusun or Tisosun beside Mufenex, or Vuzazen or Litizen beside Debusun, at equal sizes: ms of the
     prefill of one prompt and of a decode step."""
     import torch
     from xinfer_amd.engine import ModelRunner, StepEntry, build_model
@@ -302,7 +306,7 @@ def design_compare(spec: str, layers, steps: int, warmup: int, batch: int, conte
                        "token_side": {"dim": TISOSUN_SIDE}, "max_positions": 2 * context,
                        "layers": [{"type": kinds[i % 4][0], "mixer": kinds[i % 4][1], "mlp": mlp} for i in range(layers)]}
             return {"tisosun": tisosun, "mufenex": mufenex}
-        if name in ("debusun", "vuzazen"):
+        if name in ("debusun", "vuzazen", "litizen"):
             # layers of a latent, windowed attention, a state space and windowed attention again, in turn; all of them
             # are one span that runs once, so that the start of a pass is in the step
             rot = dict(dims=z["dim"], base=500000.0)
@@ -319,6 +323,20 @@ def design_compare(spec: str, layers, steps: int, warmup: int, batch: int, conte
                        "max_positions": 2 * context, "loop": {"start": 0, "stop": layers, "times": 1},
                        "layers": [{"type": kinds[i % 4][0], "mixer": kinds[i % 4][1], "mlp": {"kind": "dense", "ff": z["ff"]}}
                                   for i in range(layers)]}
+            if name == "litizen":
+                # windowed attention, a state space, attention within chunks, a state space, in turn
+                sizes = dict(heads=z["heads"], kv_heads=z["kv_heads"], dim=z["dim"], vdim=z["vdim"], scale=z["dim"] ** -0.5,
+                             mask={"size": z["window"]})
+                lkinds = [("attention", dict(sizes, rot=rot)), ("mamba2", ssm),
+                          ("attention_2", dict(sizes, softcap=50.0, rot=dict(dims=z["dim"] // 2, base=500000.0))), ("mamba2", ssm)]
+                lmlp = mlp
+                if z["experts"]:
+                    lmlp = dict(mlp, router=dict(mlp["router"], identity=LITIZEN_IDENTITY), shared=dict(mlp["expert"]))
+                litizen = {"architecture": "Litizen", "vocab": DESIGN_VOCAB, "width": z["width"],
+                           "norm": {"eps": 1e-6, "groups": LITIZEN_GROUPS}, "canon": {"taps": LITIZEN_TAPS},
+                           "embedding": {"scale": 1.0}, "logit_softcap": 30.0, "max_positions": 2 * context,
+                           "layers": [{"type": lkinds[i % 4][0], "mixer": lkinds[i % 4][1], "mlp": lmlp} for i in range(layers)]}
+                return {"litizen": litizen, "debusun": debusun}
             if name == "debusun":
                 return {"debusun": debusun, "mufenex": mufenex}
             # Vuzazen: a latent, a memory, attention behind a convolution with mixed heads, a memory, in turn; no windows
@@ -479,10 +497,10 @@ def main() -> int:
                     help="serving workloads: read every step's tokens on the host before the next step is planned")
     ap.add_argument("--product", default=None, metavar="M,N,K[,slices[,shape]]",
                     help="time one bfloat16 product alone in the many-row tiled kernel and in the vendor library")
-    ap.add_argument("--design", default=None, metavar="mufenex[:SIZE]|lilalorn[:SIZE]|debusun[:SIZE]|tisosun[:SIZE]|vuzazen[:SIZE]",
-                    help="time another model family beside its closest one (Mufenex beside Qwen3, Lilalorn, Debusun or Tisosun beside Mufenex, Vuzazen beside Debusun) at equal sizes (a line of its own; --layers, --steps, "
+    ap.add_argument("--design", default=None, metavar="mufenex[:SIZE]|lilalorn[:SIZE]|debusun[:SIZE]|litizen[:SIZE]|tisosun[:SIZE]|vuzazen[:SIZE]",
+                    help="time another model family beside its closest one (Mufenex beside Qwen3, Lilalorn, Debusun or Tisosun beside Mufenex, Vuzazen or Litizen beside Debusun) at equal sizes (a line of its own; --layers, --steps, "
                          "--warmup, --batch, --context, --prefill-tokens and --only apply)")
-    ap.add_argument("--family", choices=["both", "debusun", "lilalorn", "mufenex", "qwen3", "tisosun", "vuzazen"], default="both",
+    ap.add_argument("--family", choices=["both", "debusun", "lilalorn", "litizen", "mufenex", "qwen3", "tisosun", "vuzazen"], default="both",
                     help="--design: time one of the two families only (for profiling)")
     ap.add_argument("--peaks", action="store_true",
                     help="also measure what this card reaches on a read-only stream of 4 GiB and on one square "

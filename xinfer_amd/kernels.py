@@ -1953,7 +1953,7 @@ def head_rows(qkv: torch.Tensor, slots: torch.Tensor, k_cache: torch.Tensor, v_c
         return q_out
     _ok(lib().xi_head_rows(_p(qkv), _code(qkv, "head_rows"), _p(slots), _p(q_out), _p(k_cache), _p(v_cache),
                            int(k_cache.shape[2]), T, nq, nkv, d, dv, int(bool(v_grouped)), _p(cos if rot else None),
-                           _p(sin if rot else None), rot, int(bool(interleaved)), _p(positions if rot else None),
+                           _p(sin if rot else None), rot, int(bool(interleaved)), _p(positions if rot or v_cos is not None else None),
                            int(bool(unit_norm)), ctypes.c_float(eps), _p(bias), _p(q_weight), _p(k_weight), ctypes.c_longlong(stride),
                            v_col, _p(v_cos), _p(v_sin), _stream()))
     return q_out
