@@ -46,6 +46,10 @@ feed-forwards of a squared relu; a table of token pairs beside the embedding) be
 of their own, of a matrix memory, and of attention behind a short convolution whose heads' scores are mixed, in turn;
 dense silu feed-forwards, or experts that see the token times its score) beside Debusun at equal sizes, which has no
 experts: at the size with experts its feed-forwards are dense of the same active width.
+`--design tisosun[:SIZE]` times the Tisosun family beside dense Mufenex, `--design litizen[:SIZE]` the Litizen family (layers
+of windowed attention whose values are its keys, of a selective state space, of attention within chunks whose values turn, and
+of the state space again; dense feed-forwards, or experts beside identity experts and a shared one) beside Debusun, whose
+feed-forwards are dense at every size.
 """
 from __future__ import annotations
 
